@@ -63,16 +63,18 @@ TUFF_EXPORT int tuff_scale_cap(float* x, long long n, float scale, float cap, hi
 
 // -------------------------------------------------------------------- RMSNorm
 // y_i = x_i * (1 / sqrt(mean_j x_j^2 + eps)) * w_i   (src/lfm25_gpu.cu:235,244).
-// `rows` (optional) gathers input rows: output row r is the norm of x[rows[r]].
+// `rows` (optional) gathers input rows: output row r is the norm of x[rows[r]]; rows of x lie ldx elements apart (they
+// may be a column range of a wider row).
 // Per-thread strided partial sums -> wave butterfly -> wave partials in order; which elements a
 // thread takes depends on d alone (multiples of 4: four neighbours a step).
 template <typename TW, typename TO, bool VEC>
 __global__ __launch_bounds__(256) void rmsnorm_kernel(const float* __restrict__ x, const TW* __restrict__ w,
-                                                      TO* __restrict__ out, const int* __restrict__ rows, int d, float eps) {
+                                                      TO* __restrict__ out, const int* __restrict__ rows, int d, long long ldx,
+                                                      float eps) {
     __shared__ float scratch[4];
     const int r = blockIdx.x;
     const long long src = rows ? rows[r] : r;
-    const float* xr = x + src * (long long)d;
+    const float* xr = x + src * ldx;
     TO* o = out + (long long)r * d;
     float ss = 0.f;
     if (VEC) {
@@ -101,12 +103,14 @@ __global__ __launch_bounds__(256) void rmsnorm_kernel(const float* __restrict__ 
 }
 
 TUFF_EXPORT int tuff_rmsnorm(const float* x, const void* w, int w_dt, void* out, int out_dt,
-                             const int* rows, int n_rows, int d, float eps, hipStream_t stream) {
+                             const int* rows, int n_rows, int d, long long ldx, float eps, hipStream_t stream) {
     if (n_rows <= 0) return 0;
+    if (d <= 0 || ldx < d) return -2;
+    const bool vec = d % 4 == 0 && ldx % 4 == 0 && (uintptr_t)x % 16 == 0;
     dim3 grid(n_rows), block(256);
 #define LAUNCH(TW, TO) do { \
-        if (d % 4 == 0) hipLaunchKernelGGL((rmsnorm_kernel<TW, TO, true>), grid, block, 0, stream, x, (const TW*)w, (TO*)out, rows, d, eps); \
-        else hipLaunchKernelGGL((rmsnorm_kernel<TW, TO, false>), grid, block, 0, stream, x, (const TW*)w, (TO*)out, rows, d, eps); \
+        if (vec) hipLaunchKernelGGL((rmsnorm_kernel<TW, TO, true>), grid, block, 0, stream, x, (const TW*)w, (TO*)out, rows, d, ldx, eps); \
+        else hipLaunchKernelGGL((rmsnorm_kernel<TW, TO, false>), grid, block, 0, stream, x, (const TW*)w, (TO*)out, rows, d, ldx, eps); \
     } while (0)
     if (w_dt == DT_F32 && out_dt == DT_F32) LAUNCH(float, float);
     else if (w_dt == DT_F32 && out_dt == DT_BF16) LAUNCH(float, bf16_t);
@@ -228,15 +232,23 @@ TUFF_EXPORT int tuff_dyt(const float* x, const float* w, const float* b, const f
 }
 
 // ------------------------------------------------------------- activations
-// kind: 0 silu, 1 gelu (tanh form), 2 relu squared, 3 tanh, 4 sigmoid; evaluated in float32.
+// kind: 0 silu, 1 gelu (tanh form), 2 relu squared, 3 tanh, 4 sigmoid, 6 gelu (exact, with erf); evaluated in float32.
+// (5 is the clamped gated form of glu_kernel below, 7 the form with parameters after this one.)
 __device__ __forceinline__ float activation(float z, int kind) {
     switch (kind) {
         case 0: return z / (1.0f + expf(-z));
         case 1: return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
         case 2: { const float r = fmaxf(z, 0.f); return r * r; }
         case 3: return tanhf(z);
+        case 6: return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f));
         default: return 1.0f / (1.0f + expf(-z));
     }
+}
+
+// xIELU with a, b > 0: z > 0: a z^2 + z / 2;  z <= 0: (1/2 + b) (e^z - 1 - z) + z / 2.
+__device__ __forceinline__ float xielu(float z, float a, float b) {
+    if (z > 0.f) return fmaf(a * z, z, 0.5f * z);
+    return fmaf(0.5f + b, expm1f(z) - z, 0.5f * z);
 }
 
 // act[t, f] = f(g) * u with g = gu[t, f], u = gu[t, F + f]: the gated product of a feed-forward whose
@@ -276,14 +288,15 @@ TUFF_EXPORT int tuff_glu(const void* gu, int in_dt, void* act, int dt, int n_tok
 
 // out[t, c] = f(in[t, c] + (col_bias ? col_bias[c] : 0)) * (row_gate ? g(row_gate[t * gate_stride]) : 1): an activation
 // (after a bias per column, where given), optionally times one number a row (g: gate_kind, or -1 for the number as
-// it is).  in and out may be the same memory.
+// it is).  in and out may be the same memory.  kind 7: xIELU, a and b the two numbers at `params`.
 template <typename TI, typename TO>
 __global__ void act_rows_kernel(const TI* __restrict__ in, TO* __restrict__ out, long long n, int N, int kind,
                                 const float* __restrict__ row_gate, int gate_stride, int gate_kind,
-                                const float* __restrict__ col_bias) {
+                                const float* __restrict__ col_bias, const float* __restrict__ params) {
     const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n) return;
-    float v = activation(to_f32(in[i]) + (col_bias ? col_bias[i % N] : 0.f), kind);
+    const float z = to_f32(in[i]) + (col_bias ? col_bias[i % N] : 0.f);
+    float v = kind == 7 ? xielu(z, params[0], params[1]) : activation(z, kind);
     if (row_gate) {
         const float g = row_gate[(i / N) * gate_stride];
         v *= gate_kind < 0 ? g : activation(g, gate_kind);
@@ -292,11 +305,13 @@ __global__ void act_rows_kernel(const TI* __restrict__ in, TO* __restrict__ out,
 }
 
 TUFF_EXPORT int tuff_act_rows(const void* in, int in_dt, void* out, int out_dt, long long rows, int N, int kind,
-                              const float* row_gate, int gate_stride, int gate_kind, const float* col_bias, hipStream_t stream) {
+                              const float* row_gate, int gate_stride, int gate_kind, const float* col_bias, const float* params,
+                              hipStream_t stream) {
     const long long n = rows * N;
     if (n <= 0) return 0;
+    if ((kind == 7) != (params != nullptr)) return -2;
     dim3 grid((unsigned)ceil_div_ll(n, 256)), block(256);
-#define LAUNCH(TI, TO) hipLaunchKernelGGL((act_rows_kernel<TI, TO>), grid, block, 0, stream, (const TI*)in, (TO*)out, n, N, kind, row_gate, gate_stride, gate_kind, col_bias)
+#define LAUNCH(TI, TO) hipLaunchKernelGGL((act_rows_kernel<TI, TO>), grid, block, 0, stream, (const TI*)in, (TO*)out, n, N, kind, row_gate, gate_stride, gate_kind, col_bias, params)
     if (in_dt == DT_F32 && out_dt == DT_F32) LAUNCH(float, float);
     else if (in_dt == DT_F32) LAUNCH(float, bf16_t);
     else if (out_dt == DT_F32) LAUNCH(bf16_t, float);

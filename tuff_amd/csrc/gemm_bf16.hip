@@ -586,7 +586,7 @@ template <int NW, int MODE, int NORM, bool EMIT, int COLS, int MT>
 __global__ __launch_bounds__(NW * WAVE) void gemm_bf16_skinny16_kernel(const void* __restrict__ Xv, const bf16_t* __restrict__ W,
                                                                        void* __restrict__ Y, int M, int N, int K,
                                                                        const float* __restrict__ norm_w, float eps,
-                                                                       const int* __restrict__ rows,
+                                                                       const int* __restrict__ rows, long long ldx,
                                                                        const float* __restrict__ ss_in, int n_ss,
                                                                        const float* __restrict__ emit_nw,
                                                                        bf16_t* __restrict__ emit_xw, float* __restrict__ emit_ss,
@@ -616,7 +616,7 @@ __global__ __launch_bounds__(NW * WAVE) void gemm_bf16_skinny16_kernel(const voi
     const int wpiece = COLS == 8 ? g * 16 + (int)(n0 % 16) + r16 : lane;
     const bool wlane = COLS == 8 ? r16 < 8 : true;
     const float* xrow = nullptr;
-    if (NORM == NORM_INSIDE && r16 < M) xrow = (const float*)Xv + (long long)(rows ? rows[r16] : r16) * K;
+    if (NORM == NORM_INSIDE && r16 < M) xrow = (const float*)Xv + (long long)(rows ? rows[r16] : r16) * ldx;
 
     // What the epilogue adds to is read now, not after the last product: a load at the end would
     // cost one more trip to memory.  (Thread t of every 256 -> element (row (t / 64) * 4 + t % 4,
@@ -1277,7 +1277,7 @@ TiledPlan plan_tiled(int M, int N, int K) {
 }
 
 struct Skinny16Extra {
-    const float* norm_w = nullptr; float eps = 0.f; const int* rows = nullptr;       // NORM_INSIDE
+    const float* norm_w = nullptr; float eps = 0.f; const int* rows = nullptr; long long ldx = 0;       // NORM_INSIDE (ldx: rows of X that far apart)
     const float* ss_in = nullptr; int n_ss = 0;                                      // NORM_SCALED (+ eps)
     const float* emit_nw = nullptr; bf16_t* emit_xw = nullptr; float* emit_ss = nullptr;   // EMIT
     ConvTail conv;                                                                   // OUT_CONV
@@ -1290,7 +1290,7 @@ int launch_skinny16(const void* X, const bf16_t* W, void* Y, int M, int N, int K
     const size_t lds = NORM == NORM_INSIDE ? (size_t)K * sizeof(float) : 0;
     const int mt = M > 16 ? 2 : 1;
 #define GO_MT(NW, COLS, MT) hipLaunchKernelGGL((gemm_bf16_skinny16_kernel<NW, MODE, NORM, EMIT, COLS, MT>), grid, dim3(NW * WAVE), lds, stream, \
-                                        X, W, Y, M, N, K, x.norm_w, x.eps, x.rows, x.ss_in, x.n_ss, x.emit_nw, x.emit_xw, x.emit_ss, \
+                                        X, W, Y, M, N, K, x.norm_w, x.eps, x.rows, x.ldx ? x.ldx : (long long)K, x.ss_in, x.n_ss, x.emit_nw, x.emit_xw, x.emit_ss, \
                                         x.conv)
 #define GO(NW, COLS) do { \
         if (mt == 1) GO_MT(NW, COLS, 1); \
@@ -1541,14 +1541,15 @@ TUFF_EXPORT int tuff_gemm_bf16(const void* X, const void* W, void* Y, int M, int
     return -3;
 }
 
-// Y (=|+=) RMSNorm(X[rows]) * W^T for M <= 16 rows: X float32 [*, K], norm_w float32 [K], rows
-// optional int32 [M].  K must be a multiple of 8 and at most 8192 (the norm weight sits in LDS).
-TUFF_EXPORT int tuff_gemm_bf16_normed(const float* X, const int* rows, const float* norm_w, float eps, const void* W,
+// Y (=|+=) RMSNorm(X[rows]) * W^T for M <= 16 rows: X float32 [*, K], rows ldx elements apart (a multiple of 4, rows on
+// 16-byte borders), norm_w float32 [K], rows optional int32 [M].  K must be a multiple of 8 and at most 8192 (the norm
+// weight sits in LDS).
+TUFF_EXPORT int tuff_gemm_bf16_normed(const float* X, const int* rows, long long ldx, const float* norm_w, float eps, const void* W,
                                       void* Y, int M, int N, int K, int mode, hipStream_t stream) {
     if (M <= 0 || N <= 0) return 0;
-    if (K % 8 != 0 || K > 8192 || M > 16) return -2;
+    if (K % 8 != 0 || K > 8192 || M > 16 || ldx < K || ldx % 4 || (uintptr_t)X % 16) return -2;
     Skinny16Extra x;
-    x.norm_w = norm_w; x.eps = eps; x.rows = rows;
+    x.norm_w = norm_w; x.eps = eps; x.rows = rows; x.ldx = ldx;
     return launch_skinny16_mode<NORM_INSIDE>(X, (const bf16_t*)W, Y, M, N, K, mode, x, stream);
 }
 

@@ -12,65 +12,69 @@
 // sigmoid(gate[t][h]): both per-head products above (W_uk as stored is [H][dim][rank]; W_uv is transposed per
 // head when it is bound).  Sums run over k in ascending order in float32, one chain a (token, head, column).
 //
-// Rotation: neighbouring pairs (2i, 2i+1) of the first `rot_dims` channels of the rotated part turn by
-// pos * inv_freq[i] (float32 angle, cosf and sinf); channels beyond rot_dims pass.
+// Rotation: neighbouring pairs (2i, 2i+1), or (`halves`) pairs (i, i + rot_dims / 2), of the first `rot_dims` channels of
+// the rotated part turn by pos * inv_freq[i] (float32 angle, cosf and sinf, once a token for all heads); channels beyond
+// rot_dims pass.
 #include "common.h"
 #include <math.h>
 
 namespace {
 constexpr int POST_THREADS = 256;
 
-template <typename T, typename TW>
+// TC: the type of the latent's projected channels (a product's float32 sums may come in as they are).  ckr null: nothing is
+// cached, only the queries' rotated parts are formed.
+template <typename T, typename TC, typename TW>
 __global__ __launch_bounds__(POST_THREADS) void latent_post_kernel(
-    const T* __restrict__ proj, int row_stride, int q_off, int ckr_off, T* __restrict__ q_lat, T* __restrict__ cache,
+    const T* __restrict__ q, long long q_row, const TC* __restrict__ ckr, long long ckr_row, T* __restrict__ q_lat, T* __restrict__ cache,
     T* __restrict__ cache_t, int page_size, const TW* __restrict__ norm_w, float eps, const float* __restrict__ inv_freq, int rot_dims,
-    const int* __restrict__ positions, const int* __restrict__ slot_mapping, int H, int dim, int rot, int rank) {
+    int halves, const int* __restrict__ positions, const int* __restrict__ slot_mapping, int H, int dim, int rot, int rank) {
     __shared__ float scratch[POST_THREADS / WAVE];
+    extern __shared__ float angles[];                                    // [rot_dims / 2] cosines, then as many sines
     const long long t = blockIdx.x;
-    const T* row = proj + t * row_stride;
     const float pos = (float)positions[t];
-    const int lat = rank + rot;
-    // the latent row: norm over the first `rank` channels
-    float ss = 0.f;
-    for (int c = threadIdx.x; c < rank; c += POST_THREADS) { const float v = to_f32(row[ckr_off + c]); ss = fmaf(v, v, ss); }
-    const float total = block_sum<POST_THREADS / WAVE>(ss, scratch);
-    const float inv = 1.0f / sqrtf(total / (float)rank + eps);
-    const long long slot = slot_mapping ? slot_mapping[t] : -1;
+    const int lat = rank + rot, turns = rot_dims / 2;
+    for (int p = threadIdx.x; p < turns; p += POST_THREADS) {
+        const float a = pos * inv_freq[p];
+        angles[p] = cosf(a);
+        angles[turns + p] = sinf(a);
+    }
+    const long long slot = ckr && slot_mapping ? slot_mapping[t] : -1;
     // cache_t: the same row once more with a channel's positions contiguous within the page,
     // [page][channel][offset], as the matrix-core attention kernels read values
     T* dst_t = nullptr;
     if (slot >= 0 && cache_t) dst_t = cache_t + (slot / page_size) * (long long)lat * page_size + slot % page_size;
+    const TC* row = ckr ? ckr + t * ckr_row : nullptr;
     if (slot >= 0) {
+        // the latent row: norm over the first `rank` channels
+        float ss = 0.f;
+        for (int c = threadIdx.x; c < rank; c += POST_THREADS) { const float v = to_f32(row[c]); ss = fmaf(v, v, ss); }
+        const float total = block_sum<POST_THREADS / WAVE>(ss, scratch);
+        const float inv = 1.0f / sqrtf(total / (float)rank + eps);
         T* dst = cache + slot * lat;
         for (int c = threadIdx.x; c < rank; c += POST_THREADS) {
-            const T v = from_f32<T>(to_f32(row[ckr_off + c]) * inv * to_f32(norm_w[c]));
+            const T v = from_f32<T>(to_f32(row[c]) * inv * to_f32(norm_w[c]));
             dst[c] = v;
             if (dst_t) dst_t[(long long)c * page_size] = v;
         }
     }
-    // rotated parts: item 0 is the shared key part, items 1..H the heads' query parts; a thread a pair
-    const int pairs = rot / 2, odd = rot % 2;
-    for (int i = threadIdx.x; i < (H + 1) * (pairs + odd); i += POST_THREADS) {
-        const int item = i / (pairs + odd), p = i % (pairs + odd);
-        const T* src = item == 0 ? row + ckr_off + rank : row + q_off + (long long)(item - 1) * (dim + rot) + dim;
-        T* dst = item == 0 ? (slot >= 0 ? cache + slot * lat + rank : nullptr) : q_lat + (t * H + (item - 1)) * lat + rank;
-        if (!dst) continue;
-        T* dt2 = item == 0 && dst_t ? dst_t + (long long)rank * page_size : nullptr;
-        if (p == pairs) {                                                // a last channel without a partner passes
-            dst[rot - 1] = src[rot - 1];
-            if (dt2) dt2[(long long)(rot - 1) * page_size] = src[rot - 1];
-            continue;
-        }
-        float u = to_f32(src[2 * p]), v = to_f32(src[2 * p + 1]);
-        if (2 * p + 1 < rot_dims) {
-            const float a = pos * inv_freq[p];
-            const float cs = cosf(a), sn = sinf(a);
-            const float u2 = u * cs - v * sn, v2 = v * cs + u * sn;
-            u = u2; v = v2;
-        }
-        dst[2 * p] = from_f32<T>(u);
-        dst[2 * p + 1] = from_f32<T>(v);
-        if (dt2) { dt2[(long long)(2 * p) * page_size] = from_f32<T>(u); dt2[(long long)(2 * p + 1) * page_size] = from_f32<T>(v); }
+    __syncthreads();                                                     // the angles are there
+    // rotated parts: item 0 is the shared key part, items 1..H the heads' query parts; a thread a pair, or a channel that passes
+    const int steps = turns + rot - rot_dims;
+    for (int i = threadIdx.x; i < (H + 1) * steps; i += POST_THREADS) {
+        const int item = i / steps, p = i % steps;
+        if (item == 0 && slot < 0) continue;
+        const T* sq = item == 0 ? nullptr : q + t * q_row + (long long)(item - 1) * (dim + rot) + dim;
+        const auto in = [&](int c) { return item == 0 ? to_f32(row[rank + c]) : to_f32(sq[c]); };
+        T* dst = item == 0 ? cache + slot * lat + rank : q_lat + (t * H + (item - 1)) * lat + rank;
+        const auto out = [&](int c, float v) {
+            dst[c] = from_f32<T>(v);
+            if (item == 0 && dst_t) dst_t[(long long)(rank + c) * page_size] = from_f32<T>(v);
+        };
+        if (p >= turns) { const int c = rot_dims + p - turns; out(c, in(c)); continue; }
+        const int cu = halves ? p : 2 * p, cv = halves ? p + turns : 2 * p + 1;
+        const float u = in(cu), v = in(cv), cs = angles[p], sn = angles[turns + p];
+        out(cu, u * cs - v * sn);
+        out(cv, v * cs + u * sn);
     }
 }
 
@@ -177,25 +181,27 @@ __global__ __launch_bounds__(256) void head_matmul_mfma_kernel(const bf16_t* __r
 }
 }  // namespace
 
-// proj [T][row_stride] of type dt holds, a token: the heads' queries [H][dim + rot] from q_off, the latent's raw
-// channels [rank] and the shared key part [rot] from ckr_off.  Writes cache row slot_mapping[t] = [norm(c) w | rotate(k)]
-// (cache [slots][rank + rot]; slot_mapping null or a negative slot: nothing is written) and q_lat[t][h][rank ..] =
-// rotate(q_rot); q_lat [T][H][rank + rot].  norm_w [rank] of type norm_dt; inv_freq float32 [rot_dims / 2].
+// q: a token's queries [H][dim + rot] of type dt, rows q_row elements apart; ckr (or null): the latent's raw channels [rank] and
+// the shared key part [rot] of type ckr_dt (dt or float32), rows ckr_row apart.  Writes cache row slot_mapping[t] =
+// [norm(c) w | rotate(k)] (cache [slots][rank + rot] of type dt; ckr or slot_mapping null, or a negative slot: nothing is
+// written) and q_lat[t][h][rank ..] = rotate(q_rot); q_lat [T][H][rank + rot].  norm_w [rank] of type norm_dt; inv_freq
+// float32 [rot_dims / 2]; halves: pairs (i, i + rot_dims / 2) turn instead of neighbours.
 // cache_t (or null): the rows once more as [pages][rank + rot][page_size], for kernels that read values that way.
-TUFF_EXPORT int tuff_latent_post(const void* proj, int row_stride, int q_off, int ckr_off, void* q_lat, void* cache,
+TUFF_EXPORT int tuff_latent_post(const void* q, long long q_row, const void* ckr, int ckr_dt, long long ckr_row, void* q_lat, void* cache,
                                  void* cache_t, int page_size, int dt,
-                                 const void* norm_w, int norm_dt, float eps, const float* inv_freq, int rot_dims,
+                                 const void* norm_w, int norm_dt, float eps, const float* inv_freq, int rot_dims, int halves,
                                  const int* positions, const int* slot_mapping, int n_tokens, int H, int dim, int rot, int rank,
                                  hipStream_t stream) {
     if (n_tokens <= 0) return 0;
-    if (H < 1 || dim < 0 || rot < 0 || rank < 1 || rot_dims < 0 || rot_dims > rot || rot_dims % 2) return -2;
+    if (H < 1 || dim < 0 || rot < 0 || rank < 1 || rot_dims < 0 || rot_dims > rot || rot_dims % 2 || rot_dims > 8192) return -2;
     if (cache_t && page_size < 1) return -2;
-#define LAUNCH(T, TW) hipLaunchKernelGGL((latent_post_kernel<T, TW>), dim3(n_tokens), dim3(POST_THREADS), 0, stream, (const T*)proj, \
-        row_stride, q_off, ckr_off, (T*)q_lat, (T*)cache, (T*)cache_t, page_size, (const TW*)norm_w, eps, inv_freq, rot_dims, positions, slot_mapping, H, dim, rot, rank)
-    if (dt == DT_F32 && norm_dt == DT_F32) LAUNCH(float, float);
-    else if (dt == DT_F32) LAUNCH(float, bf16_t);
-    else if (norm_dt == DT_F32) LAUNCH(bf16_t, float);
-    else LAUNCH(bf16_t, bf16_t);
+    if (ckr && ckr_dt != dt && ckr_dt != DT_F32) return -2;
+#define LAUNCH(T, TC, TW) hipLaunchKernelGGL((latent_post_kernel<T, TC, TW>), dim3(n_tokens), dim3(POST_THREADS), rot_dims * sizeof(float), \
+        stream, (const T*)q, q_row, (const TC*)ckr, ckr_row, (T*)q_lat, (T*)cache, (T*)cache_t, page_size, (const TW*)norm_w, eps, inv_freq, \
+        rot_dims, halves, positions, slot_mapping, H, dim, rot, rank)
+    if (dt == DT_F32) { if (norm_dt == DT_F32) LAUNCH(float, float, float); else LAUNCH(float, float, bf16_t); }
+    else if (ckr_dt == DT_F32) { if (norm_dt == DT_F32) LAUNCH(bf16_t, float, float); else LAUNCH(bf16_t, float, bf16_t); }
+    else { if (norm_dt == DT_F32) LAUNCH(bf16_t, bf16_t, float); else LAUNCH(bf16_t, bf16_t, bf16_t); }
 #undef LAUNCH
     return launch_status();
 }

@@ -2,11 +2,12 @@
 //
 // Routing: from router logits z [T][E] (float32) the `top` largest are chosen per token (the lower
 // index wins a tie); the weight of a choice is f(z): 0 sigmoid (each score on its own, not
-// renormalised), 1 softmax over the chosen.  Everything here is float32.
+// renormalised), 1 softmax over the chosen, 2 softmax over all experts (the chosen ones' shares, not renormalised).
+// Everything here is float32.
 //
 // Experts: y = W_down act(W_up x) with x the token's input, multiplied by the choice's weight before
-// (scale_input) or y after; act: 0 relu squared, 1 silu, 2 gelu (tanh form).  Gated experts have two first
-// matrices: y = W_down glu(W_gate x, W_up x) with glu(g, u) = act(g) u for the three above, or, act 3, the
+// (scale_input) or y after; act: 0 relu squared, 1 silu, 2 gelu (tanh form), 4 gelu (exact, with erf).  Gated experts have two first
+// matrices: y = W_down glu(W_gate x, W_up x) with glu(g, u) = act(g) u for the four above, or, act 3, the
 // clamped form g' sigmoid(alpha g') (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit).
 // The router may have a bias: z = W h + b.  A limited choice (sigmoid weights): the choice runs on
 // c = sigmoid(z) + correction instead of z, and only inside the `keep` groups of neighbouring experts (of `groups`
@@ -21,6 +22,7 @@ namespace {
 __device__ __forceinline__ float act_fn(float z, int act) {
     if (act == 0) { const float r = fmaxf(z, 0.f); return r * r; }
     if (act == 1) return z / (1.0f + expf(-z));
+    if (act == 4) return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f));
     return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 
@@ -56,6 +58,11 @@ __device__ void choose(const float* row, int* ids, float* wts, long long t, int 
     }
     if (weight_fn == 1)
         for (int s = 0; s < top; ++s) wts[(long long)t * top + s] /= den;
+    if (weight_fn == 2) {                              // the first choice is the largest of all: den over every expert
+        den = 0.f;
+        for (int e = 0; e < E; ++e) den += expf(row[e] - zmax);
+        for (int s = 0; s < top; ++s) wts[(long long)t * top + s] /= den;
+    }
 }
 
 // The limited choice of one token (see the head of the file).  row: its E logits; cs: E floats of scratch.

@@ -30,7 +30,7 @@ _SIGNATURES = {
         "tuff_embed_rows": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_float, _c_void_p],
         "tuff_add_bias": [_c_void_p, _c_int, _c_void_p, _c_ll, _c_int, _c_void_p],
         "tuff_scale_cap": [_c_void_p, _c_ll, _c_float, _c_float, _c_void_p],
-        "tuff_rmsnorm": [_c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_float, _c_void_p],
+        "tuff_rmsnorm": [_c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_ll, _c_float, _c_void_p],
         "tuff_swiglu": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
         "tuff_cast": [_c_void_p, _c_int, _c_void_p, _c_int, _c_ll, _c_void_p],
         "tuff_cast_bias": [_c_void_p, _c_void_p, _c_void_p, _c_int, _c_ll, _c_int, _c_void_p],
@@ -38,7 +38,7 @@ _SIGNATURES = {
         "tuff_scatter_i32": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_void_p],
         "tuff_dyt": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_void_p],
         "tuff_glu": [_c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_float, _c_float, _c_void_p],
-        "tuff_act_rows": [_c_void_p, _c_int, _c_void_p, _c_int, _c_ll, _c_int, _c_int, _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p],
+        "tuff_act_rows": [_c_void_p, _c_int, _c_void_p, _c_int, _c_ll, _c_int, _c_int, _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p],
         "tuff_pad_cols": [_c_void_p, _c_void_p, _c_int, _c_ll, _c_int, _c_int, _c_void_p],
     },
     "recurrent": {
@@ -91,7 +91,7 @@ _SIGNATURES = {
                                 _c_int, _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p],
         "tuff_gemm_bf16_conv64": [_c_void_p, _c_void_p, _c_int, _c_float, _c_void_p, _c_void_p, _c_int, _c_int, _c_int,
                                   _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p],
-        "tuff_gemm_bf16_normed": [_c_void_p, _c_void_p, _c_void_p, _c_float, _c_void_p, _c_void_p, _c_int, _c_int, _c_int,
+        "tuff_gemm_bf16_normed": [_c_void_p, _c_void_p, _c_ll, _c_void_p, _c_float, _c_void_p, _c_void_p, _c_int, _c_int, _c_int,
                                   _c_int, _c_void_p],
     },
     "rope_kv": {
@@ -125,9 +125,15 @@ _SIGNATURES = {
         "tuff_hc_step": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p,
                          _c_int, _c_int, _c_int, _c_float, _c_int, _c_void_p],
     },
+    "depth": {
+        "tuff_depth_average": [_c_void_p, _c_ll, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_float, _c_void_p, _c_void_p, _c_int, _c_void_p,
+                               _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p],
+        "tuff_norm_shift": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p,
+                            _c_void_p, _c_int, _c_int, _c_void_p],
+    },
     "latent": {
-        "tuff_latent_post": [_c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_int, _c_float,
-                             _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+        "tuff_latent_post": [_c_void_p, _c_ll, _c_void_p, _c_int, _c_ll, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_int,
+                             _c_float, _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
         "tuff_head_matmul": [_c_void_p, _c_ll, _c_ll, _c_void_p, _c_void_p, _c_ll, _c_ll, _c_void_p, _c_ll, _c_int,
                              _c_int, _c_int, _c_int, _c_int, _c_void_p],
         "tuff_head_matmul_mfma": [_c_void_p, _c_ll, _c_ll, _c_void_p, _c_void_p, _c_ll, _c_ll, _c_void_p, _c_ll,
@@ -352,14 +358,14 @@ def scale_cap(x: torch.Tensor, scale: float = 1.0, cap: float = 0.0) -> None:
 
 def rmsnorm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, eps: float,
             rows: Optional[torch.Tensor] = None) -> None:
+    """out = x[rows] / sqrt(mean(x[rows]^2) + eps) * w; x float32 [*, d], which may be a column range of a wider tensor."""
     n, d = out.shape
-    if rows is None:
-        _gpu("x", x, torch.float32, (n, d))
-    else:
-        _gpu("x", x, torch.float32, (None, d))
+    ldx = _rows_view("x", x, d)
+    if x.dtype != torch.float32 or (rows is None and x.shape[0] != n):
+        raise KernelError(f"rmsnorm: x must be float32 [{'*' if rows is not None else n}, {d}], got {x.dtype} {tuple(x.shape)}")
     _check(load("elementwise").tuff_rmsnorm(
         x.data_ptr(), _gpu("w", w, shape=(d,)), _dt(w), _gpu("out", out), _dt(out),
-        _opt("rows", rows, torch.int32, (n,)), n, d, float(eps), _stream()), "rmsnorm")
+        _opt("rows", rows, torch.int32, (n,)), n, d, ldx, float(eps), _stream()), "rmsnorm")
 
 
 def swiglu(gu: torch.Tensor, act: torch.Tensor) -> None:
@@ -409,8 +415,9 @@ def dyt(x: torch.Tensor, w: torch.Tensor, b: torch.Tensor, alpha: torch.Tensor, 
         _opt("rows", rows, torch.int32, (n,)), n, d, _stream()), "dyt")
 
 
-ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "relu2": 2, "tanh": 3, "sigmoid": 4}
+ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "relu2": 2, "tanh": 3, "sigmoid": 4, "gelu_erf": 6}
 GLU_ACTIVATIONS = dict(ACTIVATIONS, swish_clamp=5)
+PARAM_ACTIVATIONS = {"xielu": 7}             # with two positive numbers a, b: act_rows(..., params=)
 
 
 def glu(gu: torch.Tensor, act: torch.Tensor, activation: str, bias: Optional[torch.Tensor] = None, *,
@@ -427,11 +434,16 @@ def glu(gu: torch.Tensor, act: torch.Tensor, activation: str, bias: Optional[tor
 
 
 def act_rows(inp: torch.Tensor, out: torch.Tensor, activation: str, row_gate: Optional[torch.Tensor] = None,
-             gate_col: int = 0, gate_activation: Optional[str] = None, bias: Optional[torch.Tensor] = None) -> None:
+             gate_col: int = 0, gate_activation: Optional[str] = None, bias: Optional[torch.Tensor] = None,
+             params: Optional[torch.Tensor] = None) -> None:
     """out = activation(inp [+ bias]), each row times gate_activation(row_gate[row, gate_col]) where row_gate
     (float32 [rows, *]) is given (gate_activation None: the number as it is).  bias: float32 [N], a number a column,
-    added before the activation.  inp may be out."""
+    added before the activation.  inp may be out.  activation "xielu", with params float32 [2] = (a, b):
+    z > 0: a z^2 + z / 2, else (1/2 + b) (exp(z) - 1 - z) + z / 2."""
     rows, N = out.shape
+    if (activation in PARAM_ACTIVATIONS) != (params is not None):
+        raise KernelError(f"act_rows: '{activation}' {'needs' if params is None else 'takes no'} params")
+    kind = PARAM_ACTIVATIONS[activation] if params is not None else ACTIVATIONS[activation]
     _gpu("inp", inp, shape=(rows, N))
     _gpu("out", out)
     gp, stride = None, 0
@@ -441,8 +453,9 @@ def act_rows(inp: torch.Tensor, out: torch.Tensor, activation: str, row_gate: Op
             raise KernelError("act_rows: gate_col outside row_gate")
         gp, stride = row_gate.data_ptr() + 4 * gate_col, row_gate.shape[1]
     _check(load("elementwise").tuff_act_rows(
-        inp.data_ptr(), _dt(inp), out.data_ptr(), _dt(out), rows, N, ACTIVATIONS[activation], gp, stride,
-        -1 if gate_activation is None else ACTIVATIONS[gate_activation], _opt("bias", bias, torch.float32, (N,)), _stream()), "act_rows")
+        inp.data_ptr(), _dt(inp), out.data_ptr(), _dt(out), rows, N, kind, gp, stride,
+        -1 if gate_activation is None else ACTIVATIONS[gate_activation], _opt("bias", bias, torch.float32, (N,)),
+        _opt("params", params, torch.float32, (2,)), _stream()), "act_rows")
 
 
 def pad_cols(inp: torch.Tensor, width: int) -> torch.Tensor:
@@ -555,11 +568,13 @@ def gemm_normed(x: torch.Tensor, norm_w: torch.Tensor, eps: float, w: torch.Tens
                 rows: Optional[torch.Tensor] = None, accumulate: bool = False, swiglu: bool = False) -> None:
     """out (=|+=) rmsnorm(x[rows]) @ w.T in one kernel, for at most 16 rows: x float32 [*, K],
     norm_w float32 [K], w bfloat16 [N, K].  The row's 1/rms scales the result, the norm weight
-    the operand."""
+    the operand.  x may be a column range of a wider tensor (see gemm_normed_rows)."""
     K = x.shape[1]
     M = x.shape[0] if rows is None else rows.shape[0]
     N = w.shape[0]
-    _gpu("x", x, torch.float32)
+    ldx = _rows_view("x", x)
+    if x.dtype != torch.float32 or not gemm_normed_rows(x):
+        raise KernelError(f"gemm_normed: x must be float32 with rows on 16-byte borders, got {x.dtype} stride {x.stride()}")
     _gpu("norm_w", norm_w, torch.float32, (K,))
     w = _tiled(w, N, K)
     _opt("rows", rows, torch.int32, (M,))
@@ -568,8 +583,14 @@ def gemm_normed(x: torch.Tensor, norm_w: torch.Tensor, eps: float, w: torch.Tens
                           f"up to {NORMED_MAX_K}; got {M} rows, inner size {K}")
     mode = _bf16_mode(out, accumulate, swiglu, M, N)
     _check(load("gemm_bf16").tuff_gemm_bf16_normed(
-        x.data_ptr(), None if rows is None else rows.data_ptr(), norm_w.data_ptr(), float(eps), w.data_ptr(),
+        x.data_ptr(), None if rows is None else rows.data_ptr(), ldx, norm_w.data_ptr(), float(eps), w.data_ptr(),
         out.data_ptr(), M, N, K, mode, _stream()), "gemm_bf16_normed")
+
+
+def gemm_normed_rows(x: torch.Tensor) -> bool:
+    """Whether every row of x (which may be a column range of a wider tensor) starts on a 16-byte border, as gemm_normed
+    reads it."""
+    return (x.stride(0) % 4 == 0 or x.shape[0] == 1 and x.shape[1] % 4 == 0) and x.data_ptr() % 16 == 0
 
 
 _emit_layouts: dict = {}
@@ -995,27 +1016,86 @@ def hc_step(xs, *, y=None, mix=None, out_w=None, in_w=None, norm_w=None, eps: fl
                                       DT_F32 if h_out is None else _dt(h_out), p(u_out), S, T, d, float(eps), int(bool(clear_y)), _stream()), "hc_step")
 
 
+# ------------------------------------------------- sums over the layers, and the token shift
+DEPTH_MAX_DIM = 16384
+
+
+def depth_average(x, *, xs=None, w=None, norm_w=None, eps: float = 0.0, inv_out=None, h_out=None, mix=None, state=None,
+                  req_of_token=None, state_slot=None) -> None:
+    """With xs float32 [n, T, d] and w float32 [n] (None: ones): x [T, d] = sum_j w[j] xs[j]; without xs, x is read as it
+    is.  Then, with eps, either inv_out float32 [T] = 1 / sqrt(mean(x^2) + eps), or, with norm_w float32 [d], h_out [T, d] =
+    x / sqrt(mean(x^2) + eps) * norm_w.  mix float32 [d] (a step in which every request has one token): h_out = h + (s - h)
+    mix with s the request's row of state (float32 [slots, d]), which becomes h."""
+    T, d = x.shape
+    _gpu("x", x, torch.float32)
+    if d > DEPTH_MAX_DIM:
+        raise KernelError(f"depth_average: {d} channels, at most {DEPTH_MAX_DIM}")
+    n = 0
+    if xs is not None:
+        _gpu("xs", xs, torch.float32, (None, T, d))
+        n = xs.shape[0]
+        if n < 1 or xs.data_ptr() <= x.data_ptr() < xs.data_ptr() + xs.numel() * 4:
+            raise KernelError("depth_average: at least one stream, and x is none of them")
+    _opt("w", w, torch.float32, (n,))
+    if (norm_w is None) != (h_out is None) or (inv_out is not None and norm_w is not None):
+        raise KernelError("depth_average: norm_w and h_out go together, inv_out goes alone")
+    _opt("norm_w", norm_w, torch.float32, (d,))
+    _opt("h_out", h_out, None, (T, d))
+    _opt("inv_out", inv_out, torch.float32, (T,))
+    if mix is not None:
+        if h_out is None:
+            raise KernelError("depth_average: the shift goes with the norm")
+        _gpu("mix", mix, torch.float32, (d,))
+        _gpu("state", state, torch.float32, (None, d))
+        _gpu("req_of_token", req_of_token, torch.int32, (T,))
+        _gpu("state_slot", state_slot, torch.int32)
+    p = lambda t: None if t is None else t.data_ptr()
+    _check(load("depth").tuff_depth_average(
+        p(xs), T * d, n, p(w), x.data_ptr(), p(norm_w), float(eps), p(inv_out), p(h_out), DT_F32 if h_out is None else _dt(h_out),
+        p(mix), p(state) if mix is not None else None, p(req_of_token) if mix is not None else None,
+        p(state_slot) if mix is not None else None, T, d, _stream()), "depth_average")
+
+
+def norm_shift(x, inv, norm_w, mix, state, out, *, req_of_token, q_start, q_len, state_slot) -> None:
+    """The normed rows h[t] = x[t] * inv[t] * norm_w (x float32 [T, d], inv float32 [T] as depth_average leaves it) mixed
+    with the row before: out[t] = h[t] + (h[t - 1] - h[t]) * mix.  The row before a request's first token of the step is
+    its row of state (float32 [slots, d]), which becomes the request's last h of the step."""
+    T, d = x.shape
+    R = q_start.shape[0]
+    _check(load("depth").tuff_norm_shift(
+        _gpu("x", x, torch.float32), _gpu("inv", inv, torch.float32, (T,)), _gpu("norm_w", norm_w, torch.float32, (d,)),
+        _gpu("mix", mix, torch.float32, (d,)), _gpu("state", state, torch.float32, (None, d)), _gpu("out", out, shape=(T, d)), _dt(out),
+        _gpu("req_of_token", req_of_token, torch.int32, (T,)), _gpu("q_start", q_start, torch.int32, (R,)),
+        _gpu("q_len", q_len, torch.int32, (R,)), _gpu("state_slot", state_slot, torch.int32, (R,)), T, d, _stream()), "norm_shift")
+
+
 # ------------------------------------------------------------------- latent attention
-def latent_post(proj, q_lat, cache, *, q_off: int, ckr_off: int, norm_w, eps: float, inv_freq, rot_dims: int, positions,
-                slot_mapping, H: int, dim: int, rot: int, rank: int, cache_t=None) -> None:
-    """From a token's projected row proj[t] (queries [H, dim + rot] from column q_off; the latent's raw channels
-    [rank] and the shared key part [rot] from column ckr_off): the cache row [norm(c) * norm_w | rotate(k)] at
-    slot_mapping[t] (cache [pages, 1, page size, rank + rot]; slot_mapping None: no write) and the rotated query
-    parts into q_lat[t, h, rank:] (q_lat [T, H * (rank + rot)]).  Rotation of neighbouring pairs of the first rot_dims
-    channels by position * inv_freq (float32 [rot_dims / 2]).  cache_t ([pages, 1, rank + rot, page size], optional):
-    the same rows once more with a channel's positions contiguous within the page."""
+def latent_post(proj, q_lat, cache, *, q_off: int, ckr_off: Optional[int], norm_w, eps: float, inv_freq, rot_dims: int, positions,
+                slot_mapping, H: int, dim: int, rot: int, rank: int, cache_t=None, ckr=None, halves: bool = False) -> None:
+    """From a token's projected rows (queries [H, dim + rot] from column q_off of proj; the latent's raw channels
+    [rank] and the shared key part [rot] from column ckr_off of ckr, which is proj unless given and may be float32):
+    the cache row [norm(c) * norm_w | rotate(k)] at slot_mapping[t] (cache [pages, 1, page size, rank + rot];
+    slot_mapping or ckr_off None: no write, and norm_w is not read) and the rotated query parts into q_lat[t, h, rank:]
+    (q_lat [T, H * (rank + rot)]).  Rotation by position * inv_freq (float32 [rot_dims / 2]) of the first rot_dims
+    channels: neighbouring pairs, or, with halves, pairs (i, i + rot_dims / 2).  cache_t ([pages, 1, rank + rot, page
+    size], optional): the same rows once more with a channel's positions contiguous within the page."""
     T = proj.shape[0]
     dt = proj.dtype
     lat = rank + rot
     _gpu("proj", proj, shape=(T, None))
-    if q_off + H * (dim + rot) > proj.shape[1] or ckr_off + lat > proj.shape[1] or min(q_off, ckr_off) < 0:
+    ckr = proj if ckr is None else ckr
+    _gpu("ckr", ckr, shape=(T, None))
+    if ckr.dtype not in (dt, torch.float32):
+        raise KernelError(f"latent_post: latent channels of type {ckr.dtype} beside queries of {dt}")
+    if q_off + H * (dim + rot) > proj.shape[1] or q_off < 0 or (ckr_off is not None and not 0 <= ckr_off <= ckr.shape[1] - lat):
         raise KernelError("latent_post: the columns lie outside the projected row")
     _gpu("q_lat", q_lat, dt, (T, H * lat))
     if cache.dim() != 4 or cache.shape[1] != 1 or cache.shape[3] != lat:
         raise KernelError(f"latent_post: the cache must be [pages, 1, page size, {lat}], got {tuple(cache.shape)}")
     _gpu("cache", cache, dt)
     _opt("cache_t", cache_t, dt, (cache.shape[0], 1, lat, cache.shape[2]))
-    _gpu("norm_w", norm_w, shape=(rank,))
+    if ckr_off is not None:
+        _gpu("norm_w", norm_w, shape=(rank,))
     if rot_dims % 2 or not 0 <= rot_dims <= rot:
         raise KernelError(f"latent_post: {rot_dims} rotated channels of {rot}")
     if rot_dims:
@@ -1023,9 +1103,11 @@ def latent_post(proj, q_lat, cache, *, q_off: int, ckr_off: int, norm_w, eps: fl
     _gpu("positions", positions, torch.int32, (T,))
     _opt("slot_mapping", slot_mapping, torch.int32, (T,))
     _check(load("latent").tuff_latent_post(
-        proj.data_ptr(), proj.shape[1], int(q_off), int(ckr_off), q_lat.data_ptr(), cache.data_ptr(),
+        proj.data_ptr() + q_off * proj.element_size(), proj.shape[1],
+        None if ckr_off is None else ckr.data_ptr() + ckr_off * ckr.element_size(), _dt(ckr), ckr.shape[1], q_lat.data_ptr(), cache.data_ptr(),
         None if cache_t is None else cache_t.data_ptr(), cache.shape[2], _dt(proj),
-        norm_w.data_ptr(), _dt(norm_w), float(eps), inv_freq.data_ptr() if rot_dims else None, int(rot_dims),
+        None if ckr_off is None else norm_w.data_ptr(), DT_F32 if ckr_off is None else _dt(norm_w), float(eps),
+        inv_freq.data_ptr() if rot_dims else None, int(rot_dims), int(bool(halves)),
         positions.data_ptr(), None if slot_mapping is None else slot_mapping.data_ptr(), T, H, dim, rot, rank, _stream()),
         "latent_post")
 
@@ -1718,16 +1800,20 @@ def head_norm_gate(o, w, gate, out, *, H, Dv, eps, per_head_weight: bool, gate_a
 
 
 # ------------------------------------------------------------------ mixture of experts
+ROUTER_WEIGHTS = {"sigmoid": 0, "softmax": 1, "softmax_all": 2}
+
+
 def moe_route(z, ids, wts, *, E, top, weights: str = "sigmoid") -> None:
     """ids, wts [T, top]: the `top` largest of z[t, :E] (float32 [T, >= E]; the lower index wins a tie) and
-    their weights, sigmoid(z) each on its own or a softmax over the chosen."""
+    their weights: sigmoid(z) each on its own, a softmax over the chosen, or ("softmax_all") the chosen ones' shares of
+    the softmax over all E."""
     T = z.shape[0]
     _gpu("z", z, torch.float32)
     if z.dim() != 2 or z.shape[1] < E:
         raise KernelError("moe_route: z must be [tokens, >= experts]")
     _check(load("moe").tuff_moe_route(z.data_ptr(), z.shape[1], _gpu("ids", ids, torch.int32, (T, top)),
                                       _gpu("wts", wts, torch.float32, (T, top)), T, E, top,
-                                      {"sigmoid": 0, "softmax": 1}[weights], _stream()), "moe_route")
+                                      ROUTER_WEIGHTS[weights], _stream()), "moe_route")
 
 
 ROUTER_MAX_FLOATS = 16380          # hidden size + logits a token: what the router kernel keeps in LDS
@@ -1748,7 +1834,7 @@ def moe_router(h, w, z, ids, wts, *, E, top, weights: str = "sigmoid", bias=None
         raise KernelError(f"moe_router: a limited choice of {top} among {keep} of {groups} groups of {E} experts is not possible")
     _check(load("moe").tuff_moe_router(_gpu("h", h), _dt(h), _gpu("w", w, torch.float32, (N, d)), _gpu("z", z, torch.float32, (T, N)),
                                        _gpu("ids", ids, torch.int32, (T, top)), _gpu("wts", wts, torch.float32, (T, top)),
-                                       T, d, N, E, top, {"sigmoid": 0, "softmax": 1}[weights],
+                                       T, d, N, E, top, ROUTER_WEIGHTS[weights],
                                        _opt("bias", bias, torch.float32, (E,)), _opt("correction", correction, torch.float32, (E,)),
                                        int(groups), int(keep), float(scale), _stream()), "moe_router")
 
@@ -1762,7 +1848,7 @@ def moe_grouped_supported(dtype, d: int, F: int, E: int) -> bool:
     return dtype == torch.bfloat16 and d % 8 == 0 and F % 8 == 0 and 1 <= E <= 1024
 
 
-EXPERT_ACTIVATIONS = {"relu2": 0, "silu": 1, "gelu_tanh": 2, "swish_clamp": 3}
+EXPERT_ACTIVATIONS = {"relu2": 0, "silu": 1, "gelu_tanh": 2, "swish_clamp": 3, "gelu_erf": 4}
 
 
 def _expert_activation(activation: str, gated: bool, limit: float) -> int:

@@ -29,13 +29,18 @@ class _Head:
 _HEAD = _Head()
 
 
+def _any_window(spec):
+    """A declaration without its window: runs that share an entry may read windows of different widths."""
+    return dataclasses.replace(spec, window=None) if isinstance(spec, PagedKV) else spec
+
+
 class DecoderModel:
     def __init__(self, *, vocab_size: int, hidden_size: int, embedding: WeightDecl,
                  blocks: list[Block], final_norm: Norm, head: Optional[WeightDecl] = None,
                  schedule: Optional[list[LayerRun]] = None, max_positions: Optional[int] = None,
                  eos_token_id: Optional[int] = None, embedding_scale: float = 1.0,
                  logit_scale: float = 1.0, logit_softcap: Optional[float] = None, pad_hidden: bool = False,
-                 streams: Optional[int] = None):
+                 streams: Optional[int] = None, depth_average: Optional[list[WeightDecl]] = None):
         """head=None: the head is the embedding (tied), as the reference does when the file has
         no output matrix (src/lfm25_model.c:128-131).
         embedding_scale: the embedding rows are multiplied by it on their way into the residual stream.
@@ -44,13 +49,22 @@ class DecoderModel:
         pad_hidden: a hidden size that is no multiple of 8 is served in bfloat16 too, by zero columns (for a
         model all of whose parts take such a size); without it such a model is refused when it is bound.
         streams: the model keeps that many residual streams [S, T, d], all equal to the embedding at the start
-        and summed before the final norm; its blocks are then all of a kind that takes them (multi_stream)."""
+        and summed before the final norm; its blocks are then all of a kind that takes them (multi_stream).
+        depth_average: one weight a run, [i + 2] for run i: with X_0 the embedding and X_(i+1) what run i makes of its
+        input, what goes on after run i is the sum of weight[j] X_j, j = 0 .. i + 1."""
         self.pad_hidden = bool(pad_hidden)
         self.streams = None if streams is None else int(streams)
         if self.streams is not None and (self.streams < 1 or not all(getattr(b, "multi_stream", False) for b in blocks)):
             raise ValueError("a model with several residual streams needs at least one and blocks that take them")
         if self.streams is None and any(getattr(b, "multi_stream", False) for b in blocks):
             raise ValueError("a block over several residual streams in a model that keeps one")
+        self.depth_decls = None if depth_average is None else list(depth_average)
+        if self.depth_decls is not None:
+            if self.streams is not None or not blocks or not all(hasattr(b, "enter") for b in blocks):
+                raise ValueError("sums over the layers go with one residual stream and blocks that enter through them")
+            runs = schedule if schedule is not None else [LayerRun(i) for i in range(len(blocks))]
+            if [tuple(w.shape) for w in self.depth_decls] != [(i + 2,) for i in range(len(runs))] or any(r.reinject for r in runs):
+                raise ValueError("sums over the layers need a weight of i + 2 numbers for every run i, and no reinjection")
         #: every block hands the next one its first normed input (Block.carries_norm): the kernel that adds a block's
         #: last output into the stream also reads the stream for whoever comes next
         self.carries = bool(blocks) and all(getattr(b, "carries_norm", False) for b in blocks)
@@ -83,8 +97,13 @@ class DecoderModel:
         self.cache_specs: dict = {}
         self._run_entries: list = []             # per run: (the mixer declares a tuple, its entry ids)
         written: dict = {}
-        for r in self.schedule:
+        self._run_states: list = []              # per run: the entry id of what the block itself keeps, or None
+        for i, r in enumerate(self.schedule):
             specs, several = cache_specs_of(self.blocks[r.block].mixer)
+            own = self.blocks[r.block].block_state() if hasattr(self.blocks[r.block], "block_state") else None
+            self._run_states.append(None if own is None else ("run", i))
+            if own is not None:
+                self.cache_specs[("run", i)] = own
             ids = tuple((r.cache, j) for j in range(len(specs))) if several else (r.cache,) * len(specs)
             if r.writes:
                 if r.cache in written:
@@ -94,11 +113,17 @@ class DecoderModel:
             else:
                 if r.cache not in written:
                     raise ValueError(f"a run reads cache entry {r.cache} before any run writes it")
-                if written[r.cache] != specs:
+                same = lambda a, b: len(a) == len(b) and all(_any_window(u) == _any_window(v) for u, v in zip(a, b))
+                if not same(written[r.cache], specs):
                     raise ValueError(f"a run reads cache entry {r.cache} of another shape: "
                                      f"{written[r.cache]} vs {specs}")
                 if any(isinstance(s_, FixedState) for s_ in specs):
                     raise ValueError("a fixed-size state cannot be shared between runs")
+                # the entry keeps what the widest window of its runs reads
+                for e, spec in zip(ids, specs):
+                    kept = self.cache_specs[e]
+                    if kept.window is not None and (spec.window is None or spec.window > kept.window):
+                        self.cache_specs[e] = dataclasses.replace(kept, window=spec.window)
             self._run_entries.append((several, ids))
         self.embedding: Optional[torch.Tensor] = None
         self.head: Optional[torch.Tensor] = None
@@ -109,6 +134,7 @@ class DecoderModel:
         for b in self.blocks:
             decls += b.weight_decls()
         decls += self.final_norm.weight_decls()
+        decls += self.depth_decls or []
         if self.head_decl is not None:
             decls.append(self.head_decl)
         seen, out = set(), []
@@ -120,7 +146,7 @@ class DecoderModel:
         return out
 
     def kernel_modules(self) -> list[str]:
-        mods = ["elementwise"]
+        mods = ["elementwise"] + (["depth"] if self.depth_decls is not None else [])
         for b in self.blocks:
             mods += b.kernel_modules()
         mods += self.final_norm.kernel_modules()
@@ -155,6 +181,8 @@ class DecoderModel:
             b.bind(weights, rt)
         self.final_norm.bind(weights, rt)
         self._head_cast: Optional[torch.Tensor] = None
+        if self.depth_decls is not None:
+            self.depth_w = [weights[w.name].float().contiguous() for w in self.depth_decls]
         if self.streams is not None:
             self._ones = torch.ones(self.streams, dtype=torch.float32, device=rt.device)
         if self.head.dtype != rt.dtype and self.head.dtype != torch.float32:
@@ -182,6 +210,8 @@ class DecoderModel:
         if self.streams is not None:
             x = self._forward_streams(ctx, cache_views)
             return self._finish(x, ctx, False, False)
+        if self.depth_decls is not None:
+            return self._finish(self._forward_depth(ctx, cache_views), ctx, *self._head_fused(ctx))
         x = torch.empty(ctx.T, self.hidden_size, dtype=torch.float32, device=rt.device)
         ops.embed_rows(self.embedding, ctx.tokens, x, self.embedding_scale)
         x0 = None
@@ -196,18 +226,40 @@ class DecoderModel:
             block = self.blocks[run.block]
             if run.reinject:
                 ops.post_norm_add(x, extra=x0)
+            own = {} if self._run_states[i] is None else {"state": cache_views[self._run_states[i]]}
             if getattr(block, "takes_next_norm", False):
                 if i + 1 < len(self.schedule):
                     nb = self.blocks[self.schedule[i + 1].block]
                     nxt = nb.first_norm_consumer() if hasattr(nb, "first_norm_consumer") else None
                 else:
                     nxt = (self.final_norm, _HEAD) if head_fused and all_rows else None
-                block.forward(x, ctx, self._views_of(i, cache_views), run.writes, next_norm=nxt)
+                block.forward(x, ctx, self._views_of(i, cache_views), run.writes, next_norm=nxt, **own)
             else:
-                block.forward(x, ctx, self._views_of(i, cache_views), run.writes)
+                block.forward(x, ctx, self._views_of(i, cache_views), run.writes, **own)
             if self.on_layer is not None:
                 self.on_layer(i, x)
         return self._finish(x, ctx, head_fused, all_rows)
+
+    def _forward_depth(self, ctx, cache_views) -> torch.Tensor:
+        """The layers of a model with sums over the layers; returns the last sum, float32 [T, d].  One buffer holds the
+        embedding and every run's stream: a run's place starts as its input, its sublayers add into it, and what stands
+        there then is its result X_(i+1), so nothing is copied.  The kernel that sums the results also norms the sum for
+        the next run's mixer."""
+        last = len(self.schedule) - 1
+        xs = torch.empty(last + 3, ctx.T, self.hidden_size, dtype=torch.float32, device=self.rt.device)
+        ops.embed_rows(self.embedding, ctx.tokens, xs[0], self.embedding_scale)
+        for i, run in enumerate(self.schedule):
+            block, x = self.blocks[run.block], xs[i + 1]
+            state = cache_views[self._run_states[i]] if self._run_states[i] is not None else None
+            h = block.enter(x, ctx, state, xs=xs[:i + 1], w=self.depth_w[i - 1] if i else None)
+            if self.on_layer is not None and i:
+                self.on_layer(i - 1, x)
+            block.forward(x, ctx, self._views_of(i, cache_views), run.writes, h=h)
+        x = xs[last + 2]
+        ops.depth_average(x, xs=xs[:last + 2], w=self.depth_w[last])
+        if self.on_layer is not None:
+            self.on_layer(last, x)
+        return x
 
     def _forward_carry(self, x, x0, ctx, cache_views) -> torch.Tensor:
         """The layers of a model whose blocks hand each other their first normed input.  The kernel that adds a block's

@@ -80,6 +80,9 @@ def _register_builtin() -> None:
     from ..config.kinelix import KinelixConfig
     from .kinelix import build_kinelix
     register_architecture(KinelixConfig.architecture, KinelixConfig, build_kinelix)
+    from ..config.kisutar import KisutarConfig
+    from .kisutar import build_kisutar
+    register_architecture(KisutarConfig.architecture, KisutarConfig, build_kisutar)
 
 
 _register_builtin()

@@ -206,6 +206,12 @@ class Block(Part):
 
     mixer: Mixer
 
+    def block_state(self):
+        """None, or the FixedState that the arrangement itself keeps per request, beside what its mixer declares; every
+        run of the block has one of its own (also a run that only reads another's cache), and forward() gets its view as
+        `state`."""
+        return None
+
     def forward(self, x, ctx, cache, write_cache: bool = True) -> None:
         raise NotImplementedError
 

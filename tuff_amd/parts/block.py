@@ -7,6 +7,9 @@ with the residual stream x in float32.  A feed-forward of None leaves out the se
 ParallelBlock has one norm whose output both sublayers read:
     h = norm(x);  x += mixer(h) + ffn(h)
 
+TokenShiftBlock is the pre-norm layer whose mixer reads each row mixed with the row before it, channel by channel:
+    h = norm1(x);  x += mixer(h + (h' - h) shift), h' the previous token's h;  x += ffn(norm2(x))
+
 SandwichBlock norms a sublayer on both sides:
     x += m * norm1b(mixer(norm1(x)));  x += m * norm2b(ffn(norm2(x)))
 
@@ -23,7 +26,7 @@ from typing import Optional
 import torch
 
 from ..csrc import ops
-from .base import BLOCKS, Block, FeedForward, Mixer, Norm, Runtime, WeightDecl
+from .base import BLOCKS, Block, FeedForward, FixedState, Mixer, Norm, Runtime, WeightDecl
 from .norm import LayerNorm, RMSNorm
 
 
@@ -66,9 +69,26 @@ class PreNormBlock(Block):
         """(norm, part that consumes it) at the head of the block, for the block before this one."""
         return self.norm1, self.mixer
 
-    def forward(self, x, ctx, cache, write_cache: bool = True, next_norm=None) -> None:
-        """next_norm: (norm, consumer) that will read x right after this block, or None."""
-        h = self._normed(self.norm1, x, self.mixer)
+    def enter(self, x, ctx, state, xs, w):
+        """For a model whose layers read weighted sums of all earlier ones: x = sum of w[j] xs[j] (xs [n, T, d]), and what
+        the mixer reads of it.  state: None."""
+        h = self.rt.empty(*x.shape)
+        if isinstance(self.norm1, RMSNorm):
+            ops.depth_average(x, xs=xs, w=w, norm_w=self.norm1.weight_f32, eps=self.norm1.eps, h_out=h)
+            return h
+        ops.depth_average(x, xs=xs, w=w)
+        return self.norm1.forward(x)
+
+    def forward(self, x, ctx, cache, write_cache: bool = True, next_norm=None, h=None) -> None:
+        """next_norm: (norm, consumer) that will read x right after this block, or None.  h: the mixer's input where
+        enter() has already run."""
+        if h is not None:
+            self._sublayers(h, x, ctx, cache, write_cache, next_norm)
+            return
+        self._sublayers(self._normed(self.norm1, x, self.mixer), x, ctx, cache, write_cache, next_norm)
+
+    def _sublayers(self, h, x, ctx, cache, write_cache, next_norm) -> None:
+        """h: what the mixer reads."""
         after = self._hand_over(self.mixer, (self.norm2, self.ffn) if self.ffn is not None else next_norm)
         self.mixer.forward(h, ctx, cache, x, write_cache, **after)
         if self.ffn is not None:
@@ -100,6 +120,61 @@ class PreNormBlock(Block):
         if consumer.accepts_pending_norm and hasattr(norm, "pending"):
             return norm.pending(x)
         return norm.forward(x)
+
+
+@BLOCKS.register("token_shift")
+class TokenShiftBlock(PreNormBlock):
+    """The pre-norm layer with a token shift: what the mixer reads is h + (h' - h) * shift, element by element, with h =
+    norm1(x) in float32 and h' the previous token's h (zeros for the first token).  The last h of a request is state of
+    the block's own, beside whatever its mixer keeps (block_state); it is float32 and formed by the same operations in
+    every kernel, so a token's input does not depend on how its sequence was cut into steps.  norm1 is an RMS norm.
+    names: checkpoint name 'shift' [d].
+
+    In a model whose layers read weighted sums of all earlier ones (DecoderModel's depth_average) one kernel forms the
+    sum, its norm and, for single tokens, the shift (enter)."""
+    def __init__(self, norm1: Norm, mixer: Mixer, norm2: Optional[Norm] = None, ffn: Optional[FeedForward] = None, *,
+                 names: dict[str, str]):
+        super().__init__(norm1, mixer, norm2, ffn)
+        if not isinstance(norm1, RMSNorm):
+            raise ValueError("the norm before a token shift is an RMS norm (it runs inside the shift's kernels)")
+        self.names = dict(names)
+
+    def weight_decls(self):
+        return super().weight_decls() + [WeightDecl(self.names["shift"], (self.norm1.dim,), "around:0.5")]
+
+    def kernel_modules(self):
+        return super().kernel_modules() + ["depth"]
+
+    def block_state(self):
+        return FixedState((self.norm1.dim,))
+
+    def bind(self, weights, rt: Runtime):
+        super().bind(weights, rt)
+        self.shift = weights[self.names["shift"]].float().contiguous()
+
+    def first_norm_consumer(self):
+        return None                       # (the product before cannot leave its operand: the rows are mixed first)
+
+    def enter(self, x, ctx, state, xs=None, w=None):
+        """The mixer's input.  With xs [n, T, d], x becomes the sum of w[j] xs[j] first."""
+        T, d = x.shape
+        h = self.rt.empty(T, d)
+        n1 = self.norm1
+        if ctx.max_q_len == 1:
+            ops.depth_average(x, xs=xs, w=w, norm_w=n1.weight_f32, eps=n1.eps, h_out=h, mix=self.shift, state=state.state,
+                              req_of_token=ctx.req_of_token, state_slot=ctx.state_slot)
+            return h
+        inv = torch.empty(T, dtype=torch.float32, device=x.device)
+        ops.depth_average(x, xs=xs, w=w, eps=n1.eps, inv_out=inv)
+        ops.norm_shift(x, inv, n1.weight_f32, self.shift, state.state, h, req_of_token=ctx.req_of_token, q_start=ctx.q_start,
+                       q_len=ctx.q_len, state_slot=ctx.state_slot)
+        return h
+
+    def forward(self, x, ctx, cache, write_cache: bool = True, next_norm=None, state=None, h=None) -> None:
+        """state: the view of block_state().  h: the mixer's input where enter() has already run."""
+        if h is None:
+            h = self.enter(x, ctx, state)
+        self._sublayers(h, x, ctx, cache, write_cache, next_norm)
 
 
 @BLOCKS.register("parallel")

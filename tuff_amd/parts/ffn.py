@@ -1,7 +1,8 @@
 """Feed-forwards.
 
 GatedMLP: W_down (act(W_gate h + b_g) * (W_up h + b_u)) + b_d with act silu or the tanh form of gelu, biases optional.
-DenseMLP: W_down act(W_up h + b_u) + b_d without a gate, act the square of relu or any other of the row activations.
+DenseMLP: W_down act(W_up h + b_u) + b_d without a gate, act the square of relu or any other of the row activations, one with
+learned numbers (xIELU) among them.
 MoE: routed experts W_down act(W_up x) chosen per token by a router, and an optional shared expert.
 
 SwiGLU feed-forward: W_down (silu(W_gate h) * (W_up h)), silu(g) = g / (1 + exp(-g)).
@@ -140,15 +141,20 @@ class GatedMLP(FeedForward):
 @FEED_FORWARDS.register("dense")
 class DenseMLP(FeedForward):
     """W_down act(W_up h + b_up) + b_down: no gate.  activation: "relu2" (the square of relu), "silu", "gelu_tanh",
-    "tanh" or "sigmoid".  names: 'up' [F, d], 'down' [d, F] and, with bias=True, 'up.b' [F], 'down.b' [d]."""
+    "gelu_erf", "tanh" or "sigmoid", or "xielu" with two learned numbers p, q: z > 0: softplus(p) z^2 + z / 2, else
+    (1/2 + softplus(q)) (e^z - 1 - z) + z / 2.  names: 'up' [F, d], 'down' [d, F]; with bias=True 'up.b' [F], 'down.b'
+    [d]; with "xielu" 'act' [2] = (p, q)."""
     graph_safe = True
     records_portions = True
+    accepts_pending_norm = True
     adds_once_through_linear = True
 
     def __init__(self, hidden_size: int, ffn_dim: int, *, names: dict[str, str], activation: str = "relu2", bias: bool = False):
-        if activation not in ops.ACTIVATIONS:
+        if activation not in ops.ACTIVATIONS and activation not in ops.PARAM_ACTIVATIONS:
             raise ValueError(f"unknown activation '{activation}'")
         self.d, self.F, self.activation, self.has_bias = int(hidden_size), int(ffn_dim), activation, bool(bias)
+        self.has_params = activation in ops.PARAM_ACTIVATIONS
+        self.params = None                                           # bound: float32 [2], the activation's numbers
         if activation == "sigmoid" and self.F % 8:
             raise ValueError("a width that is no multiple of 8 needs an activation with act(0) = 0")
         self._names = dict(names)
@@ -156,6 +162,8 @@ class DenseMLP(FeedForward):
         self._decls = self.up.weight_decls() + self.down.weight_decls()
         if self.has_bias:
             self._decls += [WeightDecl(names["up.b"], (self.F,), "normal"), WeightDecl(names["down.b"], (self.d,), "normal")]
+        if self.has_params:
+            self._decls.append(WeightDecl(names["act"], (2,), "normal"))
         #: float32 [d] once bound, or None: what the feed-forward adds to every row of its output.  A block that clears the
         #: rows its sublayers add into may leave this there instead and say so (forward(bias_preloaded=True))
         self.output_bias = None
@@ -189,11 +197,14 @@ class DenseMLP(FeedForward):
         self.down.bind(weights, rt)
         self.up_bias = weights[n["up.b"]].float().contiguous() if self.has_bias else None
         self.output_bias = weights[n["down.b"]].float().contiguous() if self.has_bias else None
+        if self.has_params:
+            z = weights[n["act"]].double()
+            self.params = torch.log1p(torch.exp(-z.abs())).add(z.clamp_min(0)).float().contiguous()      # softplus, rounded once
 
     def forward(self, h, ctx, residual, next_norm=None, bias_preloaded: bool = False) -> None:
         u = self.up.forward(h, out_dtype=torch.float32)          # the activation reads the sums as they are, plus the bias
         act = self.rt.empty(u.shape[0], self.width)
-        ops.act_rows(u, act, self.activation, bias=self.up_bias)
+        ops.act_rows(u, act, self.activation, bias=self.up_bias, params=self.params)
         if self.output_bias is None or bias_preloaded:
             self.down.forward(act, accumulate_into=residual, next_norm=next_norm)
             return
@@ -207,7 +218,7 @@ class MoE(FeedForward):
 
     Router logits z = W_router h are float32 products.  The `top` largest are chosen per token (the lower
     index wins a tie).  router_weights "sigmoid": a choice's weight is sigmoid(z), each on its own; "softmax":
-    a softmax over the chosen.  scale_input: the weight multiplies the expert's input (sum_e expert_e(w_e h));
+    a softmax over the chosen; "softmax_all": its share of the softmax over all experts, not renormalised.  scale_input: the weight multiplies the expert's input (sum_e expert_e(w_e h));
     else its output.  The shared expert runs for every token and is multiplied by sigmoid(W_sg h), one number a
     token (names['shared.sg'], [1, d]); without that name it is added as it is.
     names: 'router' [E, d]; 'experts': a list of (up [F, d], down [d, F]) names; optional 'shared.up',
@@ -242,8 +253,10 @@ class MoE(FeedForward):
                 raise ValueError("a limited choice goes with sigmoid weights and no bias on the logits")
             if not 1 <= G <= 64 or self.E % G or not 1 <= keep <= G or self.top > keep * (self.E // G):
                 raise ValueError(f"top {self.top} among {keep} of {G} groups of {self.E} experts")
-        if activation not in ("relu2", "silu", "gelu_tanh", "swish_clamp"):
+        if activation not in ops.EXPERT_ACTIVATIONS:
             raise ValueError(f"unknown activation '{activation}'")
+        if router_weights not in ops.ROUTER_WEIGHTS:
+            raise ValueError(f"unknown router weights '{router_weights}'")
         self.gated, self.limit, self.alpha = bool(gated), float(limit), float(alpha)
         if activation == "swish_clamp" and (not self.gated or not self.limit > 0):
             raise ValueError("the clamped activation is for gated experts and needs a positive limit")

@@ -140,7 +140,7 @@ class Linear:
             fused = w.dtype == torch.bfloat16 and self.in_features % 8 == 0 and (
                 ops.gemm_scaled_supported(T, self.out_features, self.in_features, want_out, accumulate_into is not None)
                 if pending.pre is not None
-                else T <= ops.NORMED_MAX_ROWS and self.in_features <= ops.NORMED_MAX_K)
+                else T <= ops.NORMED_MAX_ROWS and self.in_features <= ops.NORMED_MAX_K and ops.gemm_normed_rows(pending.x))
             if not fused:
                 x, pending = pending.tensor(), None
         if pending is None:
