@@ -92,7 +92,8 @@ def _inspect(cfg, model, out=sys.stdout) -> None:
         mixer, ffn = getattr(b, "mixer", None), getattr(b, "ffn", None)
         inside = " + ".join(_part_name(p) for p in (mixer, ffn) if p is not None) or type(b).__name__
         spec = mixer.cache_spec() if hasattr(mixer, "cache_spec") else None
-        print(f"  layer {i}: {type(b).__name__}: {inside}  cache: {spec}", file=out)
+        own = b.block_state() if hasattr(b, "block_state") else None
+        print(f"  layer {i}: {type(b).__name__}: {inside}  cache: {spec}" + (f"  own state: {own}" if own is not None else ""), file=out)
     print(f"run order: {[r.block for r in model.schedule]}", file=out)
 
 
