@@ -417,6 +417,37 @@ def kinelix_config(size: str):
                              "norm": {"eps": 1e-5}, "logit_softcap": 30.0, "layers": layers})
 
 
+def kisutar_config(size: str):
+    """`--design kisutar`: latent attention in every layer (heads of 64 + 32 rotated channels, values of 64, a cache row of
+    192 + 32, queries through a row of half the width, a window of 1,024), layers 2 and 3 of every four on the rows of
+    layer 1; dense xIELU feed-forwards and experts with a shared one take turns."""
+    from tuff_amd.models.registry import config_from_dict
+    d, L, H, G, ff, E, top, eff = DESIGN_SIZES[size]
+    mlps = [{"kind": "dense", "ff": ff},
+            {"kind": "moe", "router": {"experts": E, "top": top}, "expert": {"ff": eff}, "shared": {"ff": eff}}]
+    m = {"heads": H, "dim": 64, "rot_dim": 32, "vdim": 64, "q_rank": d // 2, "kv_rank": 192, "scale": 0.1,
+         "rot": {"base": 10000.0, "dims": 32}, "mask": {"size": 1024}}
+    layers = [{"type": "latent_attention", "mixer": dict(m, **({"kv_from": i - i % 4 + 1} if i % 4 > 1 else {})), "mlp": mlps[i % 2]}
+              for i in range(L)]
+    return config_from_dict({"architecture": "Kisutar", "vocab": DESIGN_VOCAB, "width": d, "norm": {"eps": 1e-5}, "layers": layers})
+
+
+def kinelix_config_like(size: str):
+    """The Kinelix model with latent attention in every layer that kisutar_config has: as many heads of 64 + 32 channels over a
+    cache row of 224 (no rotation, no window, queries from the full width), the same layers on another's rows, gated
+    feed-forwards of two thirds of the width (the same number of weights), the same experts likewise."""
+    from tuff_amd.models.registry import config_from_dict
+    d, L, H, G, ff, E, top, eff = DESIGN_SIZES[size]
+    gated = lambda n: n * 2 // 3 // 8 * 8
+    mlps = [{"kind": "dense", "ff": gated(ff)},
+            {"kind": "moe", "router": {"experts": E, "top": top, "scale": 1.0, "groups": {"count": 1, "keep": 1}}, "expert": {"ff": gated(eff)}}]
+    m = {"heads": H, "dim": 96, "vdim": 64, "kv_rank": 224, "scale": 0.1}
+    layers = [{"type": "latent_attention", "mixer": dict(m, **({"kv_from": i - i % 4 + 1} if i % 4 > 1 else {})), "mlp": mlps[i % 2]}
+              for i in range(L)]
+    return config_from_dict({"architecture": "Kinelix", "vocab": DESIGN_VOCAB, "width": d, "embedding": {"scale": 1.0},
+                             "norm": {"eps": 1e-5}, "layers": layers})
+
+
 def lfm2_config_like(size: str, attention_every: int = 4):
     """The LFM2 model of the same width, depth, heads, vocabulary and dense feed-forward: its short-conv
     layers stand where the other design has its recurrences (attention_every 1: attention in every layer, beside a
@@ -497,22 +528,24 @@ def time_design(cfg, dtype: str, prefill_tokens: int, batch: int, context: int, 
 
 
 def run_design(args) -> dict:
-    """`--design pafodra|kugalorn|loluzen|kinelix`: that decoder at sizes that resemble a real model's layers (random weights)
-    beside the LFM2 decoder of equal width, depth and feed-forward."""
+    """`--design pafodra|kugalorn|loluzen|kinelix|kisutar`: that decoder at sizes that resemble a real model's layers (random
+    weights) beside the LFM2 decoder of equal width, depth and feed-forward (kisutar: beside the Kinelix decoder with latent
+    attention in every layer)."""
     dtype = "bfloat16" if args.dtype == "bf16" else "float32"
     classes = os.environ.get("TUFF_TRACE", "")[:1] == "1"
     design, make = args.design, {"pafodra": pafodra_config, "kugalorn": kugalorn_config, "loluzen": loluzen_config,
-                                 "kinelix": kinelix_config}[args.design]
+                                 "kinelix": kinelix_config, "kisutar": kisutar_config}[args.design]
     every = 1 if design == "loluzen" else 4
+    other, make_other = ("kinelix", kinelix_config_like) if design == "kisutar" else ("lfm2", lambda size: lfm2_config_like(size, every))
     out = {"design": design, "dtype": args.dtype, "prefill_tokens": PREFILL_TOKENS, "decode_batch": args.batch,
            "decode_context": args.design_context, "data": f"synthetic: seeded random weights (seed {SEED}), uniform random token ids",
            "sizes": {}}
     for size in args.design_sizes.split(","):
         rec = {}
-        for name, cfg in ((design, make(size)), ("lfm2", lfm2_config_like(size, every))):
+        for name, cfg in ((design, make(size)), (other, make_other(size))):
             rec[name] = time_design(cfg, dtype, PREFILL_TOKENS, args.batch, args.design_context, args.point_steps, classes)
-        rec["prefill_ratio"] = round(rec[design]["prefill_tok_s"] / rec["lfm2"]["prefill_tok_s"], 3)
-        rec["decode_ratio"] = round(rec[design]["decode_tok_s"] / rec["lfm2"]["decode_tok_s"], 3)
+        rec["prefill_ratio"] = round(rec[design]["prefill_tok_s"] / rec[other]["prefill_tok_s"], 3)
+        rec["decode_ratio"] = round(rec[design]["decode_tok_s"] / rec[other]["decode_tok_s"], 3)
         out["sizes"][size] = rec
     return out
 
@@ -595,9 +628,9 @@ def main() -> int:
     ap.add_argument("--shape", default="1.2b", choices=["1.2b"] + sorted(OTHER_SHAPES),
                     help="measure another shape of the architecture in the benchmark's place (for profiling; "
                          "its points only, no other shapes after it)")
-    ap.add_argument("--design", choices=["pafodra", "kugalorn", "loluzen", "kinelix"],
+    ap.add_argument("--design", choices=["pafodra", "kugalorn", "loluzen", "kinelix", "kisutar"],
                     help="instead of the benchmark: prefill and decode of another design at sizes that resemble a real "
-                         "model's layers, beside the LFM2 model of equal size (TUFF_TRACE=1 adds GPU time by kernel class)")
+                         "model's layers, beside the LFM2 model of equal size, kisutar beside Kinelix (TUFF_TRACE=1 adds GPU time by kernel class)")
     ap.add_argument("--design-sizes", default="1k,2k", help="with --design: which of " + ",".join(sorted(DESIGN_SIZES)))
     ap.add_argument("--design-context", type=int, default=2048, help="with --design: tokens every decoding request holds")
     ap.add_argument("--scenario", choices=sorted(SCENARIOS),
