@@ -412,6 +412,63 @@ def test_norm_shift_kernel_alone_across_cuts(gpu, d):
             assert torch.isnan(state[0]).all() and torch.isnan(state[2]).all() and torch.isnan(state[4]).all()
 
 
+@pytest.mark.parametrize("H, Hkv, hd, vd, window, copies", [(6, 1, 40, 40, 100, 1), (32, 1, 224, 224, 1024, 1), (17, 1, 136, 64, 0, 1),
+                                                           (8, 4, 64, 128, 1, 1), (40, 2, 256, 256, 300, 1), (3, 3, 8, 8, 129, 1),
+                                                           (16, 1, 128, 96, 0, 40), (32, 1, 64, 64, 700, 60)])
+def test_single_token_attention_with_float32_weights_alone(gpu, H, Hkv, hd, vd, window, copies):
+    """Tokens at positions on both sides of every border of blocks, parts, pages and windows, pages scattered among NaN,
+    a key beside the window's edge and a far one made to stand out; `copies`: enough rows that the plan takes longer parts."""
+    from tuff_amd.csrc import ops
+    g = torch.Generator().manual_seed(H + hd)
+    ps, scale = 16, 4.0 / math.sqrt(hd)
+    pos_all = [0, 1, 15, 16, 127, 128, 129, 255, 256, 700, 1023, 1024, 1500, 2047]
+    n = max(pos_all) + 1
+    blocks = -(-n // ps)
+    P = blocks + 7
+    perm = torch.randperm(P, generator=g)[:blocks]
+    K, V = (torch.randn(n, Hkv, w, generator=g).to(torch.bfloat16) for w in (hd, vd))
+    sinks, slopes = torch.randn(H, generator=g) + 1.0, torch.rand(H, generator=g) * 0.01
+    q = torch.randn(len(pos_all), H, hd, generator=g)
+    for i, p in enumerate(pos_all):                       # one head looks at the oldest key it sees, one at the newest one it does not
+        lo = max(0, p - window + 1) if window else 0
+        q[i, 0] = K[lo, 0].float() * 0.5
+        q[i, H - 1] = K[max(0, lo - 1), Hkv - 1].float() * 0.5
+    q = q.to(torch.bfloat16)
+    kc = torch.full((P, Hkv, ps, hd), float("nan"), dtype=torch.bfloat16)
+    vc = torch.full((P, Hkv, vd, ps), float("nan"), dtype=torch.bfloat16)
+    for b in range(blocks):
+        m = min(ps, n - b * ps)
+        kc[perm[b], :, :m] = K[b * ps:b * ps + m].transpose(0, 1)
+        vc[perm[b], :, :, :m] = V[b * ps:b * ps + m].permute(1, 2, 0)
+    table = torch.stack([perm, perm]).to(torch.int32)
+    want = torch.zeros(len(pos_all), H, vd, dtype=torch.float64)
+    for i, p in enumerate(pos_all):
+        lo = max(0, p - window + 1) if window else 0
+        for h in range(H):
+            kh = h // (H // Hkv)
+            s = (K[lo:p + 1, kh].double() @ q[i, h].double()) * scale - slopes[h].double() * (p - torch.arange(lo, p + 1).double())
+            top = max(float(s.max()), float(sinks[h]))
+            e = torch.exp(s - top)
+            want[i, h] = (e @ V[lo:p + 1, kh].double()) / (e.sum() + math.exp(float(sinks[h]) - top))
+    dev = lambda t: t.to(gpu).contiguous()
+    T = len(pos_all) * copies
+    pk, slots = ops.attention_single_plan(T, H, Hkv, n, window)
+    assert (pk > 128) == (copies > 1) and slots <= 64
+    out = torch.zeros(T, H * vd, device=gpu)
+    ops.attention_single(dev(q.reshape(-1, H * hd).repeat(copies, 1)), dev(kc), dev(vc), out, block_table=dev(table),
+                         req_of_token=torch.tensor([i % 2 for i in range(T)], dtype=torch.int32, device=gpu),
+                         positions=torch.tensor(pos_all * copies, dtype=torch.int32, device=gpu), H=H, Hkv=Hkv, hd=hd, vd=vd, page_size=ps,
+                         max_ctx_len=n, window=window, scale=scale, sinks=dev(sinks), slopes=dev(slopes))
+    got = out.view(copies, len(pos_all), H, vd).double().cpu()
+    err = (got - want).abs().amax(dim=(0, 2, 3))
+    assert (err < 4e-5 * float(want.abs().max())).all(), (pos_all, err)
+    # every plan: from one token to as many as there are, at contexts up to a million positions
+    for T in (1, 8, 64, 300):
+        for ctx in (1, 16, 1000, 8192, 131072, 1 << 20):
+            pk, slots = ops.attention_single_plan(T, H, Hkv, ctx, window)
+            assert pk % 128 == 0 and 1 <= slots <= 64 and pk * (slots if not window else max(slots, 2)) >= min(ctx, window or ctx)
+
+
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("H, dk, dr, rank, dims", [(3, 8, 8, 24, 8), (1, 5, 6, 11, 4), (20, 16, 64, 192, 64), (2, 4, 2, 8, 0)])
 def test_latent_post_kernel_halves_separate_rows_and_readers(gpu, H, dk, dr, rank, dims, dtype):

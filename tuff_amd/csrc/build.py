@@ -35,6 +35,7 @@ MODULES = {
     "attention": "attention.hip",
     "attention_mfma": "attention_mfma.hip",
     "attention_prefill": "attention_prefill.hip",
+    "attention_single": "attention_single.hip",
     "shortconv": "shortconv.hip",
     "recurrent": "recurrent.hip",
     "moe": "moe.hip",

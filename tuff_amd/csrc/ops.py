@@ -114,6 +114,12 @@ _SIGNATURES = {
         "tuff_head_mix_gate": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int,
                                _c_void_p],
     },
+    "attention_single": {
+        "tuff_attention_single_plan": [_c_int, _c_int, _c_int, _c_int, _c_int, ctypes.POINTER(_c_int), ctypes.POINTER(_c_int)],
+        "tuff_attention_single": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p,
+                                  _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void_p, _c_void_p,
+                                  _c_int, _c_int, _c_void_p],
+    },
     "postnorm": {
         "tuff_post_norm_add": [_c_void_p, _c_void_p, _c_void_p, _c_float, _c_float, _c_void_p, _c_void_p, _c_float, _c_void_p,
                                _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p],
@@ -1441,6 +1447,61 @@ def attention_decode_exact(q, k_cache, v_cache, out, *, block_table, req_of_toke
         block_table.data_ptr(), block_table.shape[1], req_of_token.data_ptr(), positions.data_ptr(), T, H, Hkv, hd, vd, page_size,
         int(window or 0), float(scale), ptr(sinks), ptr(slopes), ptr(r1), ptr(r2), ptr(talk), ptr(gates), gate_stride, n_parts,
         _stream()), "attention_decode_exact")
+
+
+def attention_single_supported(dtype, hd: int, vd: int, page_size: int) -> bool:
+    return (dtype == torch.bfloat16 and hd % 8 == 0 and vd % 8 == 0 and 8 <= min(hd, vd) and max(hd, vd) <= 256 and page_size % 16 == 0)
+
+
+_single_plans: dict = {}
+
+
+def attention_single_plan(T: int, H: int, Hkv: int, max_ctx_len: int, window: int) -> tuple:
+    """(keys a part, parts a token) of attention_single for T tokens."""
+    key = (T, H, Hkv, max_ctx_len, window)
+    if key not in _single_plans:
+        if len(_single_plans) > 4096:
+            _single_plans.clear()
+        pk, n = _c_int(0), _c_int(0)
+        _check(load("attention_single").tuff_attention_single_plan(T, H, Hkv, max_ctx_len, window, ctypes.byref(pk), ctypes.byref(n)),
+               "attention_single_plan")
+        _single_plans[key] = (int(pk.value), int(n.value))
+    return _single_plans[key]
+
+
+def attention_single(q, k_cache, v_cache, out, *, block_table, req_of_token, positions, H, Hkv, hd, vd, page_size, max_ctx_len,
+                     window=0, scale=None, sinks=None, slopes=None) -> None:
+    """Single tokens over the bfloat16 cache on the matrix cores with float32-precise softmax weights (each goes through
+    the products as two bfloat16 numbers).  out [T, H * vd], bfloat16 or float32.  sinks, slopes: float32 [H] or None, as for
+    attention_general."""
+    T = q.shape[0]
+    if not attention_single_supported(q.dtype, hd, vd, page_size):
+        raise KernelError(f"attention_single: bfloat16, head sizes that are multiples of 8 up to 256 (got {hd}, {vd}) and a page size "
+                          f"that is a multiple of 16 (got {page_size})")
+    _gpu("q", q, torch.bfloat16, (T, H * hd))
+    _gpu("out", out, shape=(T, H * vd))
+    P = k_cache.shape[0]
+    _gpu("k_cache", k_cache, torch.bfloat16, (P, Hkv, page_size, hd))
+    _gpu("v_cache", v_cache, torch.bfloat16, (P, Hkv, vd, page_size))
+    _opt("sinks", sinks, torch.float32, (H,))
+    _opt("slopes", slopes, torch.float32, (H,))
+    _gpu("block_table", block_table, torch.int32)
+    if block_table.dim() != 2 or block_table.shape[1] * page_size < int(max_ctx_len):
+        raise KernelError("attention_single: block_table must be [requests, blocks] and cover the longest context")
+    _gpu("req_of_token", req_of_token, torch.int32, (T,))
+    _gpu("positions", positions, torch.int32, (T,))
+    if H % Hkv:
+        raise KernelError("attention_single: the query heads must be a multiple of the kv heads")
+    if scale is None:
+        scale = 1.0 / math.sqrt(hd)
+    part_keys, n_slots = attention_single_plan(T, H, Hkv, int(max_ctx_len), int(window or 0))
+    ws_o = torch.empty(T * H * n_slots * vd, dtype=torch.float32, device=q.device)
+    ws_ml = torch.empty(T * H * n_slots * 2, dtype=torch.float32, device=q.device)
+    ptr = lambda x: None if x is None else x.data_ptr()
+    _check(load("attention_single").tuff_attention_single(
+        q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(), _dt(out), ws_o.data_ptr(), ws_ml.data_ptr(),
+        block_table.data_ptr(), block_table.shape[1], req_of_token.data_ptr(), positions.data_ptr(), T, H, Hkv, hd, vd, page_size,
+        int(window or 0), float(scale), ptr(sinks), ptr(slopes), part_keys, n_slots, _stream()), "attention_single")
 
 
 def attention_prefill_wide_supported(dtype, hd: int, vd: int, page_size: int) -> bool:

@@ -86,6 +86,14 @@ class PagedAttention:
         G = self.H // self.Hkv
         log_distance, talk = getattr(self, "log_distance", None), getattr(self, "talk", None)
         exact = getattr(self, "exact_weights", False)
+        if (exact and log_distance is None and talk is None and gates is None and ctx.max_q_len == 1
+                and ops.attention_single_supported(q.dtype, self.hd, self.vd, cache.page_size)):
+            # single tokens with float32 weights on the matrix cores
+            ops.attention_single(q, cache.k, cache.v, o, block_table=g.block_table, req_of_token=ctx.req_of_token,
+                                 positions=ctx.positions, H=self.H, Hkv=self.Hkv, hd=self.hd, vd=self.vd, page_size=cache.page_size,
+                                 max_ctx_len=ctx.max_ctx_len, window=self.window or 0, scale=self.scale, sinks=self.sinks,
+                                 slopes=self.slopes)
+            return
         if self._single_tokens_exact(q.dtype, ctx, cache.page_size):
             ops.attention_decode_exact(q, cache.k, cache.v, o, block_table=g.block_table, req_of_token=ctx.req_of_token,
                                        positions=ctx.positions, H=self.H, Hkv=self.Hkv, hd=self.hd, vd=self.vd,
@@ -228,7 +236,7 @@ class AttentionMixer(Mixer, PagedAttention):
         return decls
 
     def kernel_modules(self):
-        mods = ["rope_kv", "attention", "attention_mfma", "attention_prefill"]
+        mods = ["rope_kv", "attention", "attention_mfma", "attention_prefill"] + (["attention_single"] if self.exact_weights else [])
         if self.K >= 1:
             mods.append("recurrent")
         if self.position is not None:

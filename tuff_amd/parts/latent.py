@@ -108,7 +108,8 @@ class LatentAttentionMixer(Mixer, PagedAttention):
         return decls
 
     def kernel_modules(self):
-        return ["latent", "attention"] + (["elementwise"] if self.q_rank is not None else []) + (["attention_mfma", "attention_prefill"] if self.twice else [])
+        return ["latent", "attention"] + (["elementwise"] if self.q_rank is not None else []) + (
+            ["attention_mfma", "attention_prefill"] + (["attention_single"] if self.exact_weights else []) if self.twice else [])
 
     def cache_spec(self):
         if self.twice:
