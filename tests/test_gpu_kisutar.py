@@ -469,6 +469,32 @@ def test_single_token_attention_with_float32_weights_alone(gpu, H, Hkv, hd, vd, 
             assert pk % 128 == 0 and 1 <= slots <= 64 and pk * (slots if not window else max(slots, 2)) >= min(ctx, window or ctx)
 
 
+@pytest.mark.parametrize("hd, vd", [(136, 64), (192, 128), (160, 136), (192, 192), (200, 192), (224, 192), (232, 40), (256, 192), (208, 208), (64, 256)])
+def test_prompt_attention_of_every_tile_width_against_the_single_token_kernel(gpu, hd, vd):
+    """The prompt kernel's tiles come in several widths: a portion's rows against the same rows taken one by one, with and
+    without a window, sinks beside."""
+    from tuff_amd.csrc import ops
+    g = torch.Generator().manual_seed(hd + vd)
+    H, T, past, ps = 5, 150, 83, 16
+    n = T + past
+    P = -(-n // ps)
+    dev = lambda t: t.to(gpu).contiguous()
+    q = dev(torch.randn(T, H * hd, generator=g).to(torch.bfloat16))
+    k = dev(torch.randn(P, 1, ps, hd, generator=g).to(torch.bfloat16))
+    v = dev(torch.randn(P, 1, vd, ps, generator=g).to(torch.bfloat16))
+    table = torch.randperm(P, generator=g).to(torch.int32)[None].to(gpu)
+    sinks = dev(torch.randn(H, generator=g))
+    for window in (0, 70):
+        kw = dict(H=H, Hkv=1, hd=hd, vd=vd, page_size=ps, max_ctx_len=n, window=window, scale=2.0 / math.sqrt(hd), sinks=sinks, block_table=table)
+        a, b = (torch.zeros(T, H * vd, dtype=torch.bfloat16, device=gpu) for _ in range(2))
+        nb = ops.attention_prefill_block_columns(max(hd, vd)) // 16
+        ops.attention_prefill_wide(q, k, v, a, blocks=torch.from_numpy(ops.query_blocks([T], H, nb, [n])).to(gpu),
+                                   req_info=torch.tensor([[0, T, past, n]], dtype=torch.int32, device=gpu), **kw)
+        ops.attention_single(q, k, v, b, req_of_token=torch.zeros(T, dtype=torch.int32, device=gpu),
+                             positions=torch.arange(past, n, dtype=torch.int32, device=gpu), **kw)
+        assert torch.isfinite(a).all() and (a.float() - b.float()).abs().max() < 1e-2 * float(b.float().abs().max()), window
+
+
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("H, dk, dr, rank, dims", [(3, 8, 8, 24, 8), (1, 5, 6, 11, 4), (20, 16, 64, 192, 64), (2, 4, 2, 8, 0)])
 def test_latent_post_kernel_halves_separate_rows_and_readers(gpu, H, dk, dr, rank, dims, dtype):
@@ -494,9 +520,9 @@ def test_latent_post_kernel_halves_separate_rows_and_readers(gpu, H, dk, dr, ran
     want_row = torch.cat([plain.rms_norm(raw[:, 5:5 + rank].double(), nw.double(), eps), turned(raw[:, 5 + rank:].double())], dim=1)
     want_q = torch.stack([turned(q[:, h * (dk + dr) + dk:(h + 1) * (dk + dr)].double()) for h in range(H)], dim=1)
     tol = 2e-4 if dtype == torch.float32 else 2e-2
-    for reader in (False, True):
+    for reader, t_ch in ((False, lat), (False, rank), (True, lat)):
         cache = torch.full((pages, 1, ps, lat), 7.0, dtype=dtype, device=gpu)
-        cache_t = torch.full((pages, 1, lat, ps), 7.0, dtype=dtype, device=gpu)
+        cache_t = torch.full((pages, 1, t_ch, ps), 7.0, dtype=dtype, device=gpu)
         q_lat = torch.full((T, H * lat), 5.0, dtype=dtype, device=gpu)
         ops.latent_post(dev(q), q_lat, cache, q_off=0, ckr=dev(raw), ckr_off=None if reader else 5, norm_w=None if reader else dev(nw), eps=eps,
                         inv_freq=dev(inv_freq.float()) if dims else None, rot_dims=dims, halves=True, positions=dev(pos),
@@ -509,7 +535,7 @@ def test_latent_post_kernel_halves_separate_rows_and_readers(gpu, H, dk, dr, ran
         if not reader:
             assert (flat[slots.long()] - want_row).abs().max() < tol * max(1.0, float(want_row.abs().max()))
             untouched[slots.long()] = False
-            assert torch.equal(cache_t.transpose(2, 3), cache)
+            assert torch.equal(cache_t.transpose(2, 3), cache[..., :t_ch])
         assert (flat[untouched] == 7.0).all()
 
 

@@ -323,12 +323,12 @@ def test_declared_tensors_and_caches():
     assert "l3.mlp.shared.up" not in decls and "l1.mlp.act" not in decls
     # a paged entry a writer, kept for the widest window of the runs that read it; a row of state for every run
     layout = CacheLayout.from_specs(model.cache_specs)
-    assert layout.paged == {0: PagedKV(1, 40, 48), 1: PagedKV(1, 40, None), 4: PagedKV(1, 24, 16)}
+    assert layout.paged == {0: PagedKV(1, 40, 48, 32), 1: PagedKV(1, 40, None, 24), 4: PagedKV(1, 24, 16, 16)}
     assert model.schedule[3].cache == 0 and not model.schedule[3].writes
     assert layout.states == {("run", i): FixedState((64,)) for i in range(5)}
     # a reader with a narrower window leaves the writer's
     plain_model = build_model(config_from_dict(copy.deepcopy(su.S_WIDE)))
-    assert plain_model.cache_specs[1] == PagedKV(1, 80, None) and plain_model.cache_specs[0] == PagedKV(1, 64, 40)
+    assert plain_model.cache_specs[1] == PagedKV(1, 80, None, 48) and plain_model.cache_specs[0] == PagedKV(1, 64, 40, 48)
 
 
 def test_a_model_with_sums_over_its_layers_refuses_what_does_not_go_with_them():

@@ -24,7 +24,7 @@
 // multiple of 16, head size a multiple of 8.
 //
 // The wide form of the kernel (EX) adds: values of another width than the keys (V [page][kv_head][vd][offset];
-// the tiles are as wide as the wider of the two and the narrower one's missing channels are zeros); a
+// the tiles are at least as wide as the rows and missing channels are zeros); a
 // logarithmic distance penalty r1_h * ln(1 + r2_h * (position - key)) off the scaled score; weights that keep
 // float32's precision through the matrix cores (a weight p goes in as two bfloat16 numbers, p rounded and
 // what the rounding left, in two products); and every query head's weights applied to the values of every kv
@@ -59,7 +59,8 @@ struct WideArgs {
     float* out_wide;            // all_v: float32 [token][head][kv head][vd]
 };
 
-template <int HDP, int NBW, int AHEAD, bool EX>
+// HDP, VDP: the channels of a key and of a value in the tiles, multiples of 32.
+template <int HDP, int NBW, int AHEAD, bool EX, int VDP>
 __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     bf16_t* __restrict__ out, const int* __restrict__ block_table, int max_blocks,
@@ -68,12 +69,12 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     int seg_keys, float* __restrict__ ws_o, float* __restrict__ ws_ml, const float* __restrict__ sinks,
     const float* __restrict__ slopes, WideArgs wide) {
     constexpr int KC = HDP / 32;          // 32-wide chunks of the head dimension
-    constexpr int DB = HDP / 16;          // 16-wide blocks of output channels
+    constexpr int DB = VDP / 16;          // 16-wide blocks of output channels
     constexpr int HC = HDP / 8;           // 16-byte chunks of a K row
     constexpr int KROW = HDP + 8;         // bf16 a K row in LDS (padded like V^T rows)
-    constexpr int KBUF = STEP * KROW, VBUF = HDP * VROW;
+    constexpr int KBUF = STEP * KROW, VBUF = VDP * VROW;
     constexpr int KPT = STEP * HC / NT;   // 16-byte pieces of K a thread copies a step
-    constexpr int VPT = HDP * 8 / NT;     // and of V^T
+    constexpr int VPT = VDP * 8 / NT;     // and of V^T
     constexpr int CB = 4 * NBW * 16;      // columns of a workgroup
     extern __shared__ __attribute__((aligned(16))) bf16_t lds[];
     bf16_t* Ks = lds;                     // [2][KBUF]
@@ -188,7 +189,7 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     bf16x8 kreg[AHEAD][KPT], vreg[AHEAD][VPT];
     int k_gran[KPT], k_key[KPT], k_off[KPT], k_lds[KPT], v_gran[VPT], v_key[VPT], v_off[VPT], v_lds[VPT];
     bool k_ok[KPT], v_ok[VPT];
-    static_assert((16 * HC) % WAVE == 0 && (2 * HDP) % WAVE == 0 && NT % WAVE == 0, "a wave's pieces lie in one granule");
+    static_assert((16 * HC) % WAVE == 0 && (2 * VDP) % WAVE == 0 && NT % WAVE == 0, "a wave's pieces lie in one granule");
 #pragma unroll
     for (int i = 0; i < KPT; ++i) {
         const int id = tid + i * NT, key = id / HC, c = id % HC;
@@ -200,14 +201,14 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     }
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
-        const int id = tid + i * NT, c8 = id / HDP, dim = id % HDP;      // lanes run over the channels
+        const int id = tid + i * NT, c8 = id / VDP, dim = id % VDP;      // lanes run over the channels
         v_gran[i] = __builtin_amdgcn_readfirstlane(c8 / 2);
         v_key[i] = c8 * 8;
         v_off[i] = dim * page_size + (c8 % 2) * 8;
         v_ok[i] = dim < vd;
         v_lds[i] = dim * VROW + c8 * 8;
     }
-    const bool whole_rows = hd == HDP && vd == HDP;
+    const bool whole_rows = hd == HDP && vd == VDP;
     const unsigned page_stride = (unsigned)(Hkv * page_size * hd);       // elements of a page in the key cache (the host checks that it fits)
     const unsigned head_off = (unsigned)(kvh * page_size * hd);          // this kv head's share of it
     const unsigned page_stride_v = (unsigned)(Hkv * page_size * vd);     // the same of the value cache
@@ -484,13 +485,13 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     }
 }
 
-template <int HDP, int NBW, int AHEAD, bool EX = false>
+template <int HDP, int NBW, int AHEAD, bool EX = false, int VDP = HDP>
 int launch(dim3 grid, hipStream_t stream, const bf16_t* q, const bf16_t* kc, const bf16_t* vc, bf16_t* out,
            const int* bt, int max_blocks, const int2* blk, const int4* req_info,
            int H, int Hkv, int hd, int ps, int window, float scale_log2e, int seg_keys, float* ws_o, float* ws_ml,
            const float* sinks, const float* slopes, WideArgs wide = WideArgs{0, nullptr, nullptr, 0, nullptr}) {
-    auto kern = attn_prefill_kernel<HDP, NBW, AHEAD, EX>;
-    constexpr int lds = 2 * (STEP * (HDP + 8) + HDP * VROW) * 2;
+    auto kern = attn_prefill_kernel<HDP, NBW, AHEAD, EX, VDP>;
+    constexpr int lds = 2 * (STEP * (HDP + 8) + VDP * VROW) * 2;
     static bool set = false;
     if (!set) {
         if (hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds) != hipSuccess) return -1;
@@ -578,13 +579,17 @@ TUFF_EXPORT int tuff_attention_prefill_wide(const void* q, const void* k_cache, 
     const float sl = scale * 1.4426950408889634f;
     const WideArgs wide{vd, log_r1, log_r2, all_v, all_v ? (float*)out : nullptr};
     const int widest = max(hd, vd);
-#define GO(HDP, NBW, AHEAD) return launch<HDP, NBW, AHEAD, true>(grid, stream, (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, \
+#define GO(HDP, NBW, AHEAD, VDP) return launch<HDP, NBW, AHEAD, true, VDP>(grid, stream, (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, \
         (bf16_t*)out, block_table, max_blocks, (const int2*)blk, (const int4*)req_info, H, Hkv, hd, page_size, window, sl, 0, nullptr, \
         nullptr, sinks, slopes, wide)
-    if (widest <= 32) GO(32, 2, 3);
-    else if (widest <= 64) GO(64, 2, 2);
-    else if (widest <= 96) GO(96, 2, 2);
-    else if (widest <= 128) GO(128, 2, 2);
-    else GO(256, 2, 1);
+    if (widest <= 32) GO(32, 2, 3, 32);
+    else if (widest <= 64) GO(64, 2, 2, 64);
+    else if (widest <= 96) GO(96, 2, 2, 96);
+    else if (widest <= 128) GO(128, 2, 2, 128);
+    else if (hd <= 192 && vd <= 128) GO(192, 2, 1, 128);       // wide rows: tiles no wider than they need be
+    else if (hd <= 192 && vd <= 192) GO(192, 2, 1, 192);
+    else if (hd <= 224 && vd <= 192) GO(224, 2, 1, 192);
+    else if (vd <= 192) GO(256, 2, 1, 192);
+    else GO(256, 2, 1, 256);
 #undef GO
 }

@@ -26,8 +26,8 @@ constexpr int POST_THREADS = 256;
 template <typename T, typename TC, typename TW>
 __global__ __launch_bounds__(POST_THREADS) void latent_post_kernel(
     const T* __restrict__ q, long long q_row, const TC* __restrict__ ckr, long long ckr_row, T* __restrict__ q_lat, T* __restrict__ cache,
-    T* __restrict__ cache_t, int page_size, const TW* __restrict__ norm_w, float eps, const float* __restrict__ inv_freq, int rot_dims,
-    int halves, const int* __restrict__ positions, const int* __restrict__ slot_mapping, int H, int dim, int rot, int rank) {
+    T* __restrict__ cache_t, int t_channels, int page_size, const TW* __restrict__ norm_w, float eps, const float* __restrict__ inv_freq,
+    int rot_dims, int halves, const int* __restrict__ positions, const int* __restrict__ slot_mapping, int H, int dim, int rot, int rank) {
     __shared__ float scratch[POST_THREADS / WAVE];
     extern __shared__ float angles[];                                    // [rot_dims / 2] cosines, then as many sines
     const long long t = blockIdx.x;
@@ -39,10 +39,10 @@ __global__ __launch_bounds__(POST_THREADS) void latent_post_kernel(
         angles[turns + p] = sinf(a);
     }
     const long long slot = ckr && slot_mapping ? slot_mapping[t] : -1;
-    // cache_t: the same row once more with a channel's positions contiguous within the page,
-    // [page][channel][offset], as the matrix-core attention kernels read values
+    // cache_t: the row's first t_channels channels (rank or all of them) once more with a channel's positions contiguous
+    // within the page, [page][channel][offset], as the matrix-core attention kernels read values
     T* dst_t = nullptr;
-    if (slot >= 0 && cache_t) dst_t = cache_t + (slot / page_size) * (long long)lat * page_size + slot % page_size;
+    if (slot >= 0 && cache_t) dst_t = cache_t + (slot / page_size) * (long long)t_channels * page_size + slot % page_size;
     const TC* row = ckr ? ckr + t * ckr_row : nullptr;
     if (slot >= 0) {
         // the latent row: norm over the first `rank` channels
@@ -68,7 +68,7 @@ __global__ __launch_bounds__(POST_THREADS) void latent_post_kernel(
         T* dst = item == 0 ? cache + slot * lat + rank : q_lat + (t * H + (item - 1)) * lat + rank;
         const auto out = [&](int c, float v) {
             dst[c] = from_f32<T>(v);
-            if (item == 0 && dst_t) dst_t[(long long)(rank + c) * page_size] = from_f32<T>(v);
+            if (item == 0 && dst_t && t_channels == lat) dst_t[(long long)(rank + c) * page_size] = from_f32<T>(v);
         };
         if (p >= turns) { const int c = rot_dims + p - turns; out(c, in(c)); continue; }
         const int cu = halves ? p : 2 * p, cv = halves ? p + turns : 2 * p + 1;
@@ -186,18 +186,19 @@ __global__ __launch_bounds__(256) void head_matmul_mfma_kernel(const bf16_t* __r
 // [norm(c) w | rotate(k)] (cache [slots][rank + rot] of type dt; ckr or slot_mapping null, or a negative slot: nothing is
 // written) and q_lat[t][h][rank ..] = rotate(q_rot); q_lat [T][H][rank + rot].  norm_w [rank] of type norm_dt; inv_freq
 // float32 [rot_dims / 2]; halves: pairs (i, i + rot_dims / 2) turn instead of neighbours.
-// cache_t (or null): the rows once more as [pages][rank + rot][page_size], for kernels that read values that way.
+// cache_t (or null): the rows' first t_channels channels (rank, or rank + rot) once more as [pages][t_channels][page_size],
+// for kernels that read values that way.
 TUFF_EXPORT int tuff_latent_post(const void* q, long long q_row, const void* ckr, int ckr_dt, long long ckr_row, void* q_lat, void* cache,
-                                 void* cache_t, int page_size, int dt,
+                                 void* cache_t, int t_channels, int page_size, int dt,
                                  const void* norm_w, int norm_dt, float eps, const float* inv_freq, int rot_dims, int halves,
                                  const int* positions, const int* slot_mapping, int n_tokens, int H, int dim, int rot, int rank,
                                  hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (H < 1 || dim < 0 || rot < 0 || rank < 1 || rot_dims < 0 || rot_dims > rot || rot_dims % 2 || rot_dims > 8192) return -2;
-    if (cache_t && page_size < 1) return -2;
+    if (cache_t && (page_size < 1 || (t_channels != rank && t_channels != rank + rot))) return -2;
     if (ckr && ckr_dt != dt && ckr_dt != DT_F32) return -2;
 #define LAUNCH(T, TC, TW) hipLaunchKernelGGL((latent_post_kernel<T, TC, TW>), dim3(n_tokens), dim3(POST_THREADS), rot_dims * sizeof(float), \
-        stream, (const T*)q, q_row, (const TC*)ckr, ckr_row, (T*)q_lat, (T*)cache, (T*)cache_t, page_size, (const TW*)norm_w, eps, inv_freq, \
+        stream, (const T*)q, q_row, (const TC*)ckr, ckr_row, (T*)q_lat, (T*)cache, (T*)cache_t, t_channels, page_size, (const TW*)norm_w, eps, inv_freq, \
         rot_dims, halves, positions, slot_mapping, H, dim, rot, rank)
     if (dt == DT_F32) { if (norm_dt == DT_F32) LAUNCH(float, float, float); else LAUNCH(float, float, bf16_t); }
     else if (ckr_dt == DT_F32) { if (norm_dt == DT_F32) LAUNCH(bf16_t, float, float); else LAUNCH(bf16_t, float, bf16_t); }

@@ -138,7 +138,7 @@ _SIGNATURES = {
                             _c_void_p, _c_int, _c_int, _c_void_p],
     },
     "latent": {
-        "tuff_latent_post": [_c_void_p, _c_ll, _c_void_p, _c_int, _c_ll, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_int,
+        "tuff_latent_post": [_c_void_p, _c_ll, _c_void_p, _c_int, _c_ll, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_int,
                              _c_float, _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
         "tuff_head_matmul": [_c_void_p, _c_ll, _c_ll, _c_void_p, _c_void_p, _c_ll, _c_ll, _c_void_p, _c_ll, _c_int,
                              _c_int, _c_int, _c_int, _c_int, _c_void_p],
@@ -1083,8 +1083,9 @@ def latent_post(proj, q_lat, cache, *, q_off: int, ckr_off: Optional[int], norm_
     the cache row [norm(c) * norm_w | rotate(k)] at slot_mapping[t] (cache [pages, 1, page size, rank + rot];
     slot_mapping or ckr_off None: no write, and norm_w is not read) and the rotated query parts into q_lat[t, h, rank:]
     (q_lat [T, H * (rank + rot)]).  Rotation by position * inv_freq (float32 [rot_dims / 2]) of the first rot_dims
-    channels: neighbouring pairs, or, with halves, pairs (i, i + rot_dims / 2).  cache_t ([pages, 1, rank + rot, page
-    size], optional): the same rows once more with a channel's positions contiguous within the page."""
+    channels: neighbouring pairs, or, with halves, pairs (i, i + rot_dims / 2).  cache_t ([pages, 1, rank + rot or
+    rank, page size], optional): the rows, or their first `rank` channels, once more with a channel's positions contiguous
+    within the page."""
     T = proj.shape[0]
     dt = proj.dtype
     lat = rank + rot
@@ -1099,7 +1100,9 @@ def latent_post(proj, q_lat, cache, *, q_off: int, ckr_off: Optional[int], norm_
     if cache.dim() != 4 or cache.shape[1] != 1 or cache.shape[3] != lat:
         raise KernelError(f"latent_post: the cache must be [pages, 1, page size, {lat}], got {tuple(cache.shape)}")
     _gpu("cache", cache, dt)
-    _opt("cache_t", cache_t, dt, (cache.shape[0], 1, lat, cache.shape[2]))
+    _opt("cache_t", cache_t, dt, (cache.shape[0], 1, None, cache.shape[2]))
+    if cache_t is not None and cache_t.shape[2] not in (rank, lat):
+        raise KernelError(f"latent_post: cache_t must hold {rank} or {lat} channels a page, got {tuple(cache_t.shape)}")
     if ckr_off is not None:
         _gpu("norm_w", norm_w, shape=(rank,))
     if rot_dims % 2 or not 0 <= rot_dims <= rot:
@@ -1111,7 +1114,7 @@ def latent_post(proj, q_lat, cache, *, q_off: int, ckr_off: Optional[int], norm_
     _check(load("latent").tuff_latent_post(
         proj.data_ptr() + q_off * proj.element_size(), proj.shape[1],
         None if ckr_off is None else ckr.data_ptr() + ckr_off * ckr.element_size(), _dt(ckr), ckr.shape[1], q_lat.data_ptr(), cache.data_ptr(),
-        None if cache_t is None else cache_t.data_ptr(), cache.shape[2], _dt(proj),
+        None if cache_t is None else cache_t.data_ptr(), 0 if cache_t is None else cache_t.shape[2], cache.shape[2], _dt(proj),
         None if ckr_off is None else norm_w.data_ptr(), DT_F32 if ckr_off is None else _dt(norm_w), float(eps),
         inv_freq.data_ptr() if rot_dims else None, int(rot_dims), int(bool(halves)),
         positions.data_ptr(), None if slot_mapping is None else slot_mapping.data_ptr(), T, H, dim, rot, rank, _stream()),

@@ -11,6 +11,7 @@ import torch
 
 from ..csrc import ops
 from ..parts.base import Block, FixedState, Norm, PagedKV, Runtime, WeightDecl, cache_specs_of
+from ..parts.norm import RMSNorm
 
 
 @dataclasses.dataclass(frozen=True)
@@ -211,7 +212,8 @@ class DecoderModel:
             x = self._forward_streams(ctx, cache_views)
             return self._finish(x, ctx, False, False)
         if self.depth_decls is not None:
-            return self._finish(self._forward_depth(ctx, cache_views), ctx, *self._head_fused(ctx))
+            x, h = self._forward_depth(ctx, cache_views)
+            return self._finish(x, ctx, False, False, h)
         x = torch.empty(ctx.T, self.hidden_size, dtype=torch.float32, device=rt.device)
         ops.embed_rows(self.embedding, ctx.tokens, x, self.embedding_scale)
         x0 = None
@@ -240,8 +242,9 @@ class DecoderModel:
                 self.on_layer(i, x)
         return self._finish(x, ctx, head_fused, all_rows)
 
-    def _forward_depth(self, ctx, cache_views) -> torch.Tensor:
-        """The layers of a model with sums over the layers; returns the last sum, float32 [T, d].  One buffer holds the
+    def _forward_depth(self, ctx, cache_views) -> tuple:
+        """The layers of a model with sums over the layers; returns the last sum, float32 [T, d], and, where every token's
+        logits are wanted and the final norm is an RMS norm, that norm of it (else None).  One buffer holds the
         embedding and every run's stream: a run's place starts as its input, its sublayers add into it, and what stands
         there then is its result X_(i+1), so nothing is copied.  The kernel that sums the results also norms the sum for
         the next run's mixer."""
@@ -256,10 +259,15 @@ class DecoderModel:
                 self.on_layer(i - 1, x)
             block.forward(x, ctx, self._views_of(i, cache_views), run.writes, h=h)
         x = xs[last + 2]
-        ops.depth_average(x, xs=xs[:last + 2], w=self.depth_w[last])
+        h = None
+        if self._head_fused(ctx)[1] and isinstance(self.final_norm, RMSNorm):
+            h = self.rt.empty(ctx.T, self.hidden_size)
+            ops.depth_average(x, xs=xs[:last + 2], w=self.depth_w[last], norm_w=self.final_norm.weight_f32, eps=self.final_norm.eps, h_out=h)
+        else:
+            ops.depth_average(x, xs=xs[:last + 2], w=self.depth_w[last])
         if self.on_layer is not None:
             self.on_layer(last, x)
-        return x
+        return x, h
 
     def _forward_carry(self, x, x0, ctx, cache_views) -> torch.Tensor:
         """The layers of a model whose blocks hand each other their first normed input.  The kernel that adds a block's
@@ -310,8 +318,9 @@ class DecoderModel:
             ops.hc_step(xs, in_w=self._ones, u_out=carry)
         return carry
 
-    def _finish(self, x, ctx, head_fused: bool, all_rows: bool) -> Optional[torch.Tensor]:
-        """The final norm and the head over x float32 [T, d]."""
+    def _finish(self, x, ctx, head_fused: bool, all_rows: bool, h=None) -> Optional[torch.Tensor]:
+        """The final norm and the head over x float32 [T, d].  h: the normed rows, where every row is wanted and they are
+        there already."""
         # which rows are wanted is a fact of the step, not of its shape: the head runs outside of what is recorded
         # (a recorder keeps the function and hands back what it returns at each replay)
         # What the last block left for the final norm is taken here, where the step's kernels are issued (or
@@ -323,7 +332,7 @@ class DecoderModel:
         out: list = []
 
         def head(c):
-            out[:] = [self._head(x, c, pre)]
+            out[:] = [self._head(x, c, pre, h)]
             return out[0]
 
         ctx.run_eagerly(head)
@@ -336,7 +345,7 @@ class DecoderModel:
         """What forward() reads of a step outside of ctx.run_eagerly and bakes into its launches: a
         recording of a step in sections is valid for steps with the same key."""
         head_fused, all_rows = self._head_fused(ctx)
-        return (ctx.T, bool(head_fused and all_rows))
+        return (ctx.T, bool((head_fused or self.depth_decls is not None) and all_rows))
 
     def _views_of(self, i: int, cache_views: dict):
         """What run i's mixer is handed as `cache`: None, a view, or a tuple of views."""
@@ -355,20 +364,20 @@ class DecoderModel:
                       or all_rows and ctx.n_logits <= ops.EMIT_MAX_ROWS))
         return fused, all_rows
 
-    def _head(self, x, ctx, pre=None) -> Optional[torch.Tensor]:
-        logits = self._head_product(x, ctx, pre)
+    def _head(self, x, ctx, pre=None, h=None) -> Optional[torch.Tensor]:
+        logits = self._head_product(x, ctx, pre, h)
         if logits is not None and (self.logit_scale != 1.0 or self.logit_softcap is not None):
             ops.scale_cap(logits, self.logit_scale, self.logit_softcap or 0.0)
         return logits
 
-    def _head_product(self, x, ctx, pre=None) -> Optional[torch.Tensor]:
-        """pre: (xw, ss), the final norm's operand and row sums as the last block's product left them, or None."""
+    def _head_product(self, x, ctx, pre=None, h=None) -> Optional[torch.Tensor]:
+        """h: the final norm's rows, where they are there already.  pre: (xw, ss), the final norm's operand and row sums as the last block's product left them, or None."""
         if ctx.n_logits == 0:
             return None
         rt = self.rt
         head_fused, all_rows = self._head_fused(ctx)
         logits = torch.empty(ctx.n_logits, self.vocab_size, dtype=torch.float32, device=rt.device)
-        if head_fused:
+        if head_fused and h is None:
             fn = self.final_norm
             if pre is not None and all_rows:
                 ops.gemm_scaled(pre[0], pre[1], fn.eps, self.head, logits)
@@ -376,7 +385,8 @@ class DecoderModel:
             if ctx.n_logits <= ops.NORMED_MAX_ROWS and self.hidden_size <= ops.NORMED_MAX_K:
                 ops.gemm_normed(x, fn.weight_f32, fn.eps, self.head, logits, rows=ctx.logit_rows)
                 return logits
-        h = self.final_norm.forward(x, rows=ctx.logit_rows)
+        if h is None:
+            h = self.final_norm.forward(x, rows=ctx.logit_rows)
         if h.dtype != self.head.dtype:
             h32 = torch.empty(h.shape, dtype=torch.float32, device=rt.device)
             ops.cast(h, h32)

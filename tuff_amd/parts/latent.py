@@ -7,8 +7,8 @@ Keys and values are expansions of one narrow row a token: with h the mixer's inp
 The cache keeps [c | k_r] and nothing else: rank + rot numbers a token, one "kv head" for all query
 heads, the row's first `rank` channels serving as the value.  Where a row is narrow enough for the
 matrix-core attention kernels (a multiple of 8, at most 256 channels) the rows are kept a second time with
-a channel's positions contiguous within the page, which is how those kernels read values; wider rows are
-kept once and go through the general kernel.  The expansions are never formed for the
+a channel's positions contiguous within the page, which is how those kernels read values (with exact_weights the
+first `rank` channels only); wider rows are kept once and go through the general kernel.  The expansions are never formed for the
 cached tokens: the query is carried into the latent space, q' = [W_uk,a^T q_plain,a | q_rot,a], attention
 runs over the cache rows as they lie, and W_uv,a is applied to the head's weighted sum of rows.
 Both per-head products (ops.head_matmul) run on the matrix cores in bfloat16 where head sizes, rank and the projected
@@ -73,7 +73,9 @@ class LatentAttentionMixer(Mixer, PagedAttention):
         self.window = int(window) if window else None
         # what PagedAttention reads: every query head against the one row a position
         self.twice = self.lat % 8 == 0 and self.lat <= 256        # rows also kept the matrix cores' way
-        self.Hkv, self.hd, self.vd = 1, self.lat, (self.lat if self.twice else self.rank)
+        # the second copy holds whole rows where the kernels take equal widths only, else the channels that are values
+        whole = self.twice and not (self.exact_weights and self.rank % 8 == 0)
+        self.Hkv, self.hd, self.vd = 1, self.lat, (self.lat if whole else self.rank)
         self.sinks = self.slopes = None
         self.names = dict(names)
         self.gated = "g" in self.names
@@ -113,7 +115,7 @@ class LatentAttentionMixer(Mixer, PagedAttention):
 
     def cache_spec(self):
         if self.twice:
-            return PagedKV(1, self.lat, self.window)
+            return PagedKV(1, self.lat, self.window, value_dim=None if self.vd == self.lat else self.vd)
         return PagedKV(1, self.lat, self.window, value_dim=self.rank, values_in_keys=True)
 
     def bind(self, weights, rt: Runtime):
@@ -156,7 +158,7 @@ class LatentAttentionMixer(Mixer, PagedAttention):
             lat_col = self.q_rank
         gate_col = lat_col + (lat if self.own_rows else 0)
         q_lat = self.rt.empty(T, H * lat)
-        o_lat = self.rt.empty(T, H * self.vd)         # (with the rows kept twice a head's sum is a whole row: its rotated part is not used)
+        o_lat = self.rt.empty(T, H * self.vd)         # (where whole rows are kept twice a head's sum is a whole row: its rotated part is not used)
         o = self.rt.empty(T, H * dv)
         # the queries' plain parts into the latent space: q'[t, a, :rank] = W_uk,a^T q_plain[t, a]
         ops.head_matmul(q, self.w_uk, q_lat, H=H, x_head=dk + dr, y_head=lat, w_nk=self.w_uk_nk)
