@@ -190,6 +190,14 @@ def ensure_built(module: str) -> str:
     return path
 
 
+def ensure_all(modules, jobs: int = 8) -> None:
+    """Compiles those of `modules` that have no current build, several at a time."""
+    from concurrent.futures import ThreadPoolExecutor
+    todo = sorted({m for m in modules if find_built(m) is None})
+    with ThreadPoolExecutor(max_workers=max(1, min(jobs, len(todo) or 1))) as ex:
+        list(ex.map(compile_module, todo))
+
+
 def build_all(force: bool = True, jobs: int = 8) -> dict[str, str]:
     """Compiles every module (in parallel).  With force=False only the missing or stale ones."""
     from concurrent.futures import ThreadPoolExecutor

@@ -116,43 +116,51 @@ __global__ __launch_bounds__(NT) void depth_average_kernel(const float* __restri
     }
 }
 
-// Thread (token, piece of V channels).  The workgroups of a request's first token are the only ones that touch its
-// state: they read it and then leave the request's last row there.
+// A thread walks SHIFT_RUN neighbouring tokens of its V channels, each row being the row before for the next one.  The
+// threads of a request's first token are the only ones that touch its state: they read it and then leave the request's
+// last row there.
+constexpr int SHIFT_RUN = 4;
+
 template <typename T, int V>
 __global__ __launch_bounds__(256) void norm_shift_kernel(const float* __restrict__ x, const float* __restrict__ inv,
                                                          const float* __restrict__ norm_w, const float* __restrict__ mix,
                                                          float* __restrict__ state, T* __restrict__ out,
                                                          const int* __restrict__ req_of_token, const int* __restrict__ q_start,
-                                                         const int* __restrict__ q_len, const int* __restrict__ state_slot, int d) {
-    const int t = blockIdx.x;
+                                                         const int* __restrict__ q_len, const int* __restrict__ state_slot, int n_tokens,
+                                                         int d) {
+    const int t0 = blockIdx.x * SHIFT_RUN, nt = min(SHIFT_RUN, n_tokens - t0);
     const int c = (blockIdx.y * 256 + threadIdx.x) * V;
     if (c >= d) return;
-    const int r = req_of_token[t];
-    const bool first = t == q_start[r];
-    float nw[V], m[V], cur[V], prev[V], o[V];
+    float nw[V], m[V], row[SHIFT_RUN + 1][V];             // row 0: the token before the run
     load_vec<V>(norm_w + c, nw);
     load_vec<V>(mix + c, m);
-    load_vec<V>(x + (long long)t * d + c, cur);
-    const float inv_t = inv[t];
-    float* st = state + (long long)state_slot[r] * d + c;
-    if (first) load_vec<V>(st, prev);
-    else {
-        load_vec<V>(x + (long long)(t - 1) * d + c, prev);
-        const float inv_p = inv[t - 1];
+    auto normed_row = [&](int t, float (&h)[V]) {
+        load_vec<V>(x + (long long)t * d + c, h);
+        const float inv_t = inv[t];
 #pragma unroll
-        for (int e = 0; e < V; ++e) prev[e] = normed(prev[e], inv_p, nw[e]);
+        for (int e = 0; e < V; ++e) h[e] = normed(h[e], inv_t, nw[e]);
+    };
+    normed_row(max(t0 - 1, 0), row[0]);                   // (used only where it is the same request's)
+#pragma unroll
+    for (int i = 0; i < SHIFT_RUN; ++i) normed_row(t0 + min(i, nt - 1), row[i + 1]);
+#pragma unroll
+    for (int i = 0; i < SHIFT_RUN; ++i) {
+        if (i >= nt) break;
+        const int t = t0 + i, r = req_of_token[t];
+        float prev[V], o[V];
+#pragma unroll
+        for (int e = 0; e < V; ++e) prev[e] = row[i][e];
+        if (t == q_start[r]) {
+            float* st = state + (long long)state_slot[r] * d + c;
+            load_vec<V>(st, prev);
+            float keep[V];
+            normed_row(t + q_len[r] - 1, keep);
+            store_vec<V>(st, keep);
+        }
+#pragma unroll
+        for (int e = 0; e < V; ++e) o[e] = shifted(row[i + 1][e], prev[e], m[e]);
+        store_as<V>(out + (long long)t * d + c, o);
     }
-#pragma unroll
-    for (int e = 0; e < V; ++e) o[e] = shifted(normed(cur[e], inv_t, nw[e]), prev[e], m[e]);
-    store_as<V>(out + (long long)t * d + c, o);
-    if (!first) return;
-    const int last = t + q_len[r] - 1;
-    float keep[V];
-    load_vec<V>(x + (long long)last * d + c, keep);
-    const float inv_l = inv[last];
-#pragma unroll
-    for (int e = 0; e < V; ++e) keep[e] = normed(keep[e], inv_l, nw[e]);
-    store_vec<V>(st, keep);
 }
 }  // namespace
 
@@ -195,9 +203,9 @@ TUFF_EXPORT int tuff_norm_shift(const float* x, const float* inv, const float* n
     if (n_tokens <= 0) return 0;
     if (d <= 0) return -2;
     const int V = d % 4 == 0 ? 4 : 1;
-    dim3 grid(n_tokens, ceil_div(d, 256 * V)), block(256);
+    dim3 grid(ceil_div(n_tokens, SHIFT_RUN), ceil_div(d, 256 * V)), block(256);
 #define GO(T, V) hipLaunchKernelGGL((norm_shift_kernel<T, V>), grid, block, 0, s, x, inv, norm_w, mix, state, (T*)out, req_of_token, \
-        q_start, q_len, state_slot, d)
+        q_start, q_len, state_slot, n_tokens, d)
     if (out_dt == DT_F32) { if (V == 4) GO(float, 4); else GO(float, 1); }
     else { if (V == 4) GO(bf16_t, 4); else GO(bf16_t, 1); }
 #undef GO

@@ -304,12 +304,41 @@ __global__ void act_rows_kernel(const TI* __restrict__ in, TO* __restrict__ out,
     out[i] = from_f32<TO>(v);
 }
 
+// The same without a row gate, four neighbouring columns a thread (N a multiple of 4, both ends on borders of their pieces).
+template <typename TI, typename TO>
+__global__ void act_rows_vec_kernel(const TI* __restrict__ in, TO* __restrict__ out, long long n4, int N, int kind,
+                                    const float* __restrict__ col_bias, const float* __restrict__ params) {
+    const long long i = ((long long)blockIdx.x * blockDim.x + threadIdx.x) * 4;
+    if (i >= n4 * 4) return;
+    typedef TI in4 __attribute__((ext_vector_type(4)));
+    typedef TO out4 __attribute__((ext_vector_type(4)));
+    const in4 v = *(const in4*)(in + i);
+    const f32x4 b = col_bias ? *(const f32x4*)(col_bias + i % N) : f32x4{0.f, 0.f, 0.f, 0.f};
+    out4 o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        const float z = to_f32((TI)v[e]) + b[e];
+        o[e] = from_f32<TO>(kind == 7 ? xielu(z, params[0], params[1]) : activation(z, kind));
+    }
+    *(out4*)(out + i) = o;
+}
+
 TUFF_EXPORT int tuff_act_rows(const void* in, int in_dt, void* out, int out_dt, long long rows, int N, int kind,
                               const float* row_gate, int gate_stride, int gate_kind, const float* col_bias, const float* params,
                               hipStream_t stream) {
     const long long n = rows * N;
     if (n <= 0) return 0;
     if ((kind == 7) != (params != nullptr)) return -2;
+    if (!row_gate && N % 4 == 0 && (uintptr_t)in % 16 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)col_bias % 16 == 0) {
+        const dim3 vgrid((unsigned)ceil_div_ll(n / 4, 256));
+#define LAUNCH(TI, TO) hipLaunchKernelGGL((act_rows_vec_kernel<TI, TO>), vgrid, dim3(256), 0, stream, (const TI*)in, (TO*)out, n / 4, N, kind, col_bias, params)
+        if (in_dt == DT_F32 && out_dt == DT_F32) LAUNCH(float, float);
+        else if (in_dt == DT_F32) LAUNCH(float, bf16_t);
+        else if (out_dt == DT_F32) LAUNCH(bf16_t, float);
+        else LAUNCH(bf16_t, bf16_t);
+#undef LAUNCH
+        return launch_status();
+    }
     dim3 grid((unsigned)ceil_div_ll(n, 256)), block(256);
 #define LAUNCH(TI, TO) hipLaunchKernelGGL((act_rows_kernel<TI, TO>), grid, block, 0, stream, (const TI*)in, (TO*)out, n, N, kind, row_gate, gate_stride, gate_kind, col_bias, params)
     if (in_dt == DT_F32 && out_dt == DT_F32) LAUNCH(float, float);

@@ -16,7 +16,7 @@ import torch
 from ..cache.manager import CacheLayout, CacheManager, OutOfPages
 from ..cache.storage import CacheStorage
 from ..config.base import ModelConfig
-from ..csrc import ops
+from ..csrc import build, ops
 from ..models.registry import build_model, load_config
 from ..parts.base import Runtime
 from ..weights.loader import load_weights
@@ -66,8 +66,10 @@ class Engine:
         self.dtype = parse_dtype(dtype)
         self.model = model
         self.rt = Runtime(self.device, self.dtype)
-        for m in model.kernel_modules() + (["gemm_f32"] if self.dtype == torch.float32 else ["gemm_bf16"]):
-            ops.load(m)                      # compile or load now, not in the middle of a step
+        modules = model.kernel_modules() + (["gemm_f32"] if self.dtype == torch.float32 else ["gemm_bf16"])
+        build.ensure_all(modules)            # compile now, not in the middle of a step
+        for m in modules:
+            ops.load(m)
         model.bind(weights, self.rt)
         # what the parts read of a step's tokens beside ids and positions (StepEntry.inputs brings it)
         self.token_inputs = tuple(model.token_inputs()) if hasattr(model, "token_inputs") else ()

@@ -111,7 +111,7 @@ class LatentAttentionMixer(Mixer, PagedAttention):
 
     def kernel_modules(self):
         return ["latent", "attention"] + (["elementwise"] if self.q_rank is not None else []) + (
-            ["attention_mfma", "attention_prefill"] + (["attention_single"] if self.exact_weights else []) if self.twice else [])
+            [] if not self.twice else ["attention_prefill", "attention_single" if self.exact_weights else "attention_mfma"])
 
     def cache_spec(self):
         if self.twice:
