@@ -589,6 +589,7 @@ TUFF_EXPORT int tuff_attention_prefill_wide(const void* q, const void* k_cache, 
     else if (hd <= 192 && vd <= 128) GO(192, 2, 1, 128);       // wide rows: tiles no wider than they need be
     else if (hd <= 192 && vd <= 192) GO(192, 2, 1, 192);
     else if (hd <= 224 && vd <= 192) GO(224, 2, 1, 192);
+    else if (widest <= 224) GO(224, 2, 1, 224);
     else if (vd <= 192) GO(256, 2, 1, 192);
     else GO(256, 2, 1, 256);
 #undef GO
