@@ -249,6 +249,41 @@ def test_peaky_attention_far_keys_in_prompts_and_in_decoding(gpu, name, dtype):
     check(name, dtype, util.plan_chunks(reqs, sizes=(15, 1, 16, 17, 2, 31, 33, 64, 63, 65)), reqs, peaky=True)
 
 
+def _drawn(seed: int) -> dict:
+    """A configuration with every size drawn, multiples of 8 in half of them."""
+    import random
+    r = random.Random(seed)
+    even = seed % 2 == 0
+    size = lambda lo, hi: (lambda v: max(8, v // 8 * 8) if even else v)(r.randint(lo, hi))
+    layers, kept = [], []
+    for i in range(r.randint(2, 5)):
+        src = r.choice(kept) if kept and r.random() < 0.4 else None
+        if src is None:
+            rank, rot, base = size(8, 300 if r.random() < 0.2 else 90), 2 * r.randint(1, 20), r.choice([30.0, 1000.0, 50000.0])
+            rot = rot // 8 * 8 + 8 if even else rot
+        else:
+            m = layers[src]["mixer"]
+            rank, rot, base = m["kv_rank"], m["rot_dim"], m["rot"]["base"]
+        window = r.choice([None, 1, r.randint(2, 40), r.randint(2, 40), r.randint(41, 200), 16, 64])
+        mixer = su.latent(r.randint(1, 12), size(3, 50), rot, size(3, 50), size(5, 70), rank, r.uniform(0.1, 0.5), window, base, src)
+        E = r.randint(1, 12)
+        mlp = r.choice([None, su.dense(size(5, 120)), su.dense(size(5, 120)), su.moe(E, r.randint(1, E), size(5, 60), r.choice([None, size(5, 60)]))])
+        if src is None:
+            kept.append(i)
+        layers.append(su.layer(mixer, mlp))
+    return su.config(size(20, 160), r.randint(30, 400), layers, eps=r.choice([1e-6, 1e-5, 1e-3]))
+
+
+@pytest.mark.parametrize("seed", range(10))
+def test_configurations_drawn_at_random(gpu, seed):
+    name = f"drawn_{seed}"
+    su.CONFIGS[name] = _drawn(seed)
+    reqs = requests(name, [61, 140, 7, 30], seed=seed)
+    for dtype in DTYPES:
+        check(name, dtype, util.plan_mixed(reqs, seed=seed, max_live=3), reqs, max_requests=3)
+        check(name, dtype, util.plan_tail(reqs, tail=16), reqs)
+
+
 # ------------------------------------------------------------ one key made to stand out
 def _bound_latent(gpu, dtype, H, rank, dr, dv, scale, window, sinks):
     """A latent mixer whose projections pick columns of its input: a row is [query row | raw latent | rotated key]; the

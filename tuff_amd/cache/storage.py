@@ -73,6 +73,8 @@ class CacheStorage:
             typed = raw.view(_STATE_DTYPES[spec.dtype])[:, :_numel(spec.shape)]
             self.views[e] = StateView(typed.view((manager.num_slots,) + tuple(spec.shape)), raw)
 
+        self._slots = [v.raw for v in self.views.values() if isinstance(v, StateView)]
+        self._slot_table = None
         if poison:
             manager.on_free = self.poison_pages
 
@@ -89,9 +91,10 @@ class CacheStorage:
                     v.v[idx] = float("nan")
 
     def zero_slot(self, slot: int) -> None:
-        for v in self.views.values():
-            if isinstance(v, StateView):
-                ops.fill_u32(v.raw[slot], 0)
+        if self._slots:
+            if self._slot_table is None:
+                self._slot_table = ops.slot_table(self._slots)
+            ops.zero_slot(self._slot_table, self._slots, slot)
 
     def nbytes(self) -> int:
         n = 0

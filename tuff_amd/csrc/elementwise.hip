@@ -191,6 +191,22 @@ TUFF_EXPORT int tuff_fill_u32(void* p, uint32_t value, long long n, hipStream_t 
     return launch_status();
 }
 
+// Clears one slot of several arrays: entry e of the table (two 64-bit words each) names an array's address and the
+// 32-bit words a slot of it has.
+__global__ void zero_slot_kernel(const long long* __restrict__ table, int slot) {
+    uint32_t* base = (uint32_t*)table[2 * blockIdx.y];
+    const long long words = table[2 * blockIdx.y + 1];
+    const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < words) base[slot * words + i] = 0u;
+}
+
+TUFF_EXPORT int tuff_zero_slot(const long long* table, int n, long long most_words, int slot, hipStream_t stream) {
+    if (n <= 0 || most_words <= 0) return 0;
+    if (n > 65535 || slot < 0) return -2;
+    hipLaunchKernelGGL(zero_slot_kernel, dim3((unsigned)ceil_div_ll(most_words, 256), n), dim3(256), 0, stream, table, slot);
+    return launch_status();
+}
+
 // -------------------------------------------------------------------- scatter
 // dst[idx[i]] = src[idx[n + i]] for i < n, bounds checked (a bad index writes nothing): token ids that
 // a sampling kernel has left on the device go into the next step's token buffer without a trip

@@ -35,6 +35,7 @@ _SIGNATURES = {
         "tuff_cast": [_c_void_p, _c_int, _c_void_p, _c_int, _c_ll, _c_void_p],
         "tuff_cast_bias": [_c_void_p, _c_void_p, _c_void_p, _c_int, _c_ll, _c_int, _c_void_p],
         "tuff_fill_u32": [_c_void_p, ctypes.c_uint32, _c_ll, _c_void_p],
+        "tuff_zero_slot": [_c_void_p, _c_int, _c_ll, _c_int, _c_void_p],
         "tuff_scatter_i32": [_c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_void_p],
         "tuff_dyt": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_void_p],
         "tuff_glu": [_c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_float, _c_float, _c_void_p],
@@ -400,6 +401,23 @@ def fill_u32(t: torch.Tensor, value: int = 0) -> None:
     if not t.is_cuda or not t.is_contiguous():
         raise KernelError("fill_u32: contiguous GPU tensor required")
     _check(load("elementwise").tuff_fill_u32(t.data_ptr(), value, t.numel(), _stream()), "fill_u32")
+
+
+def slot_table(arrays) -> torch.Tensor:
+    """The table zero_slot reads, int64 [n, 2] on the arrays' device: arrays are int32 [slots, words] each, contiguous."""
+    for a in arrays:
+        _gpu("slots", a, torch.int32)
+        if a.dim() != 2:
+            raise KernelError("slot_table: arrays must be [slots, words]")
+    return torch.tensor([[a.data_ptr(), a.shape[1]] for a in arrays], dtype=torch.int64).to(arrays[0].device)
+
+
+def zero_slot(table: torch.Tensor, arrays, slot: int) -> None:
+    """Clears row `slot` of every array (table: slot_table(arrays)) in one launch."""
+    if not 0 <= slot < min(a.shape[0] for a in arrays):
+        raise KernelError(f"zero_slot: slot {slot} is not there")
+    _check(load("elementwise").tuff_zero_slot(_gpu("table", table, torch.int64, (len(arrays), 2)), len(arrays),
+                                              max(a.shape[1] for a in arrays), int(slot), _stream()), "zero_slot")
 
 
 def scatter_i32(dst: torch.Tensor, src: torch.Tensor, idx: torch.Tensor) -> None:
