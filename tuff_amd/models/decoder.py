@@ -371,7 +371,8 @@ class DecoderModel:
         return logits
 
     def _head_product(self, x, ctx, pre=None, h=None) -> Optional[torch.Tensor]:
-        """h: the final norm's rows, where they are there already.  pre: (xw, ss), the final norm's operand and row sums as the last block's product left them, or None."""
+        """h: the final norm's rows, where they are there already.  pre: (xw, ss), the final norm's operand and row sums as
+        the last block's product left them, or None."""
         if ctx.n_logits == 0:
             return None
         rt = self.rt
