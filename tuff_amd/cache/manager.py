@@ -2,7 +2,7 @@
 request holds.
 
 Cache entries that grow a token at a time (PagedKV) are sorted into groups by what they need
-to keep: all positions, or a window of the last W.  A group has a page pool and, per request,
+to keep: all positions, or a window of the last W, with or without the sequence's first tokens besides.  A group has a page pool and, per request,
 a block table of its own; all entries of a group share the page numbering.  Entries of fixed
 size (FixedState) live in one slot per request.  Pages go back to their pool when the request
 ends or when a window has moved past them, and are handed out again (last freed, first used).
@@ -70,6 +70,7 @@ class CacheGroup:
     window: Optional[int]
     entries: list[int]            # cache entry ids in this group
     pool: PagePool
+    keep_first: int = 0           # with a window: so many of the first positions stay
 
 
 @dataclasses.dataclass
@@ -79,6 +80,7 @@ class CacheLayout:
     states: dict[int, FixedState]
     group_windows: list[Optional[int]]          # one per group
     group_of_entry: dict[int, int]
+    group_keeps: list[int] = dataclasses.field(default_factory=list)      # one per group: first positions that stay beside the window
 
     @staticmethod
     def from_specs(specs: dict[int, object]) -> "CacheLayout":
@@ -87,14 +89,15 @@ class CacheLayout:
         other = [s for s in specs.values() if s is not None and not isinstance(s, (PagedKV, FixedState))]
         if other:
             raise CacheError(f"unknown cache declaration {other[0]!r}")
-        windows: list[Optional[int]] = []
+        needs: list[tuple] = []
         group_of = {}
         for i in sorted(paged, key=lambda e: e if isinstance(e, tuple) else (e, -1)):
             w = paged[i].window
-            if w not in windows:
-                windows.append(w)
-            group_of[i] = windows.index(w)
-        return CacheLayout(paged, states, windows, group_of)
+            need = (w, paged[i].keep_first if w is not None else 0)
+            if need not in needs:
+                needs.append(need)
+            group_of[i] = needs.index(need)
+        return CacheLayout(paged, states, [w for w, _ in needs], group_of, [k for _, k in needs])
 
     def bytes_per_token(self, elem_size: int) -> int:
         return sum(s.elements_per_token * elem_size for s in self.paged.values())
@@ -120,8 +123,9 @@ class CacheManager:
         counts = [num_pages] * n_groups if isinstance(num_pages, int) else list(num_pages)
         if len(counts) != n_groups:
             raise ValueError(f"{n_groups} cache groups but {len(counts)} pool sizes")
-        self.groups = [CacheGroup(w, [e for e, g in layout.group_of_entry.items() if g == gi], PagePool(c))
-                       for gi, (w, c) in enumerate(zip(layout.group_windows, counts))]
+        keeps = layout.group_keeps or [0] * n_groups
+        self.groups = [CacheGroup(w, [e for e, g in layout.group_of_entry.items() if g == gi], PagePool(c), k)
+                       for gi, (w, c, k) in enumerate(zip(layout.group_windows, counts, keeps))]
         self._free_slots = list(range(self.num_slots - 1, -1, -1))
         self._requests: dict[Hashable, _Request] = {}
         #: debugging aid: called as on_free(group index, pages) whenever pages go back to a pool
@@ -162,12 +166,13 @@ class CacheManager:
         return self._req(req_id).slot
 
     # -------------------------------------------------------------------- pages
-    def _first_needed_block(self, group: CacheGroup, length: int) -> int:
-        """Blocks below this index hold only positions no later token of the request reads."""
+    def _passed_blocks(self, group: CacheGroup, length: int) -> tuple[int, int]:
+        """Blocks lo .. hi - 1 hold only positions no later token of the request reads: what the window has passed,
+        without the first tokens that stay."""
         if group.window is None:
-            return 0
-        first_pos = max(0, length - group.window + 1)     # earliest key the next token reads
-        return first_pos // self.page_size
+            return 0, 0
+        first_pos = max(0, length - group.window + 1)     # earliest key of the next token's window
+        return -(-group.keep_first // self.page_size), first_pos // self.page_size
 
     def pages_needed(self, req_id, n_new: int) -> list[int]:
         """Pages each group must still supply to hold n_new more tokens (after giving back
@@ -188,8 +193,8 @@ class CacheManager:
             if g.window is None:
                 out.append(0)
                 continue
-            lo = self._first_needed_block(g, r.length)
-            out.append(sum(1 for p in r.tables[gi][:lo] if p != FREED))
+            lo, hi = self._passed_blocks(g, r.length)
+            out.append(sum(1 for p in r.tables[gi][lo:hi] if p != FREED))
         return out
 
     def can_extend(self, req_id, n_new: int) -> bool:
@@ -204,12 +209,12 @@ class CacheManager:
             raise ValueError("n_new must be >= 0")
         r = self._req(req_id)
         for gi, g in enumerate(self.groups):
-            lo = self._first_needed_block(g, r.length)
-            gone = [p for p in r.tables[gi][:lo] if p != FREED]
+            lo, hi = self._passed_blocks(g, r.length)
+            gone = [p for p in r.tables[gi][lo:hi] if p != FREED]
             if gone:
                 r.arrays.pop(gi, None)
                 self._give_back(gi, gone)
-                for b in range(min(lo, len(r.tables[gi]))):
+                for b in range(lo, min(hi, len(r.tables[gi]))):
                     r.tables[gi][b] = FREED
         need = self.pages_needed(req_id, n_new)
         for n, g in zip(need, self.groups):

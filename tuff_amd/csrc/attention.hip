@@ -27,6 +27,12 @@
 // is the kv head whose values are read, out is [token][head][kv head][vd]); mixing the heads' softmax
 // weights is linear in them, so a kernel that follows forms the mixed heads from these sums.
 //
+// A window may keep the sequence's first keys: position i then also sees every key before keep_first.
+//
+// A cached key row may hold `maps` keys side by side (differential attention: several softmax maps over one kv head's
+// values).  H then counts maps, query row h (hd / maps channels) meets part h % maps of the key row, and with out_f32 the
+// sums are written in float32 for the kernel that combines them (tuff_diff_combine).
+//
 // This is the general kernel: any head size up to 640, any page size, float32 or
 // bfloat16 cache.  One wave per (token, head): lanes are keys for q.k, lanes are
 // channels for p.v.
@@ -42,7 +48,7 @@ __global__ __launch_bounds__(WAVE) void attention_general_kernel(
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ req_of_token,
     const int* __restrict__ positions, int H, int Hkv, int hd, int vd, int page_size, int window, float scale, const float* __restrict__ sinks,
     const float* __restrict__ slopes, int v_in_k, const float* __restrict__ log_r1, const float* __restrict__ log_r2,
-    int all_v) {
+    int all_v, int keep_first, int maps, int out_f32) {
     __shared__ float qs[MAX_PER_LANE * WAVE];
     __shared__ float ps[WAVE];
     __shared__ long long voff[WAVE];
@@ -51,13 +57,15 @@ __global__ __launch_bounds__(WAVE) void attention_general_kernel(
     const int pos = positions[t];
     const int lo = (window > 0) ? max(0, pos - window + 1) : 0;
     const int* table = block_table + (long long)req_of_token[t] * max_blocks;
-    const T* qrow = q + ((long long)t * H + head) * hd;
+    const int qd = hd / maps;                                 // channels of a query
+    const int k_off = (head % maps) * qd;                     // its part of the key row
+    const T* qrow = q + ((long long)t * H + head) * qd;
     const float slope = slopes ? slopes[head] : 0.f;
     const float r1 = log_r1 ? log_r1[head] : 0.f, r2 = log_r1 ? log_r2[head] : 0.f;
     const int vh = all_v ? blockIdx.z : kvh;                  // the kv head whose values are read
     const T* v_base = v_in_k ? k_cache : v_cache;
     const long long v_step = v_in_k ? 1 : page_size;          // from a value's channel to the next
-    for (int j = lane; j < hd; j += WAVE) qs[j] = to_f32(qrow[j]);
+    for (int j = lane; j < qd; j += WAVE) qs[j] = to_f32(qrow[j]);
     __syncthreads();
 
     float m = -INFINITY, l = 0.f;
@@ -65,9 +73,12 @@ __global__ __launch_bounds__(WAVE) void attention_general_kernel(
 #pragma unroll
     for (int i = 0; i < MAX_PER_LANE; ++i) acc[i] = 0.f;
 
-    for (int t0 = (lo / WAVE) * WAVE; t0 <= pos; t0 += WAVE) {
+    const int lo_tile = (lo / WAVE) * WAVE;
+    // (the tiles that hold first keys to keep, then the window's)
+    for (int t0 = keep_first > 0 ? 0 : lo_tile; t0 <= pos; t0 += WAVE) {
+        if (t0 < lo_tile && t0 >= keep_first) t0 = lo_tile;
         const int kt = t0 + lane;
-        const bool valid = kt >= lo && kt <= pos;
+        const bool valid = (kt >= lo || kt < keep_first) && kt <= pos;
         float s = -INFINITY;
         long long base = 0;
         if (valid) {
@@ -75,9 +86,9 @@ __global__ __launch_bounds__(WAVE) void attention_general_kernel(
             const long long head_base = (page * Hkv + kvh) * page_size;
             base = v_in_k ? head_base * hd + (long long)(kt % page_size) * hd      // the key's own row
                           : (page * Hkv + vh) * page_size * vd + (kt % page_size); // V: [vd][page_size], this key's column
-            const T* krow = k_cache + head_base * hd + (long long)(kt % page_size) * hd;
+            const T* krow = k_cache + head_base * hd + (long long)(kt % page_size) * hd + k_off;
             float d = 0.f;
-            for (int j = 0; j < hd; ++j) d = fmaf(qs[j], to_f32(krow[j]), d);
+            for (int j = 0; j < qd; ++j) d = fmaf(qs[j], to_f32(krow[j]), d);
             s = d * scale - slope * (float)(pos - kt);
             if (log_r1) s -= r1 * log1pf(r2 * (float)(pos - kt));
         }
@@ -121,6 +132,7 @@ __global__ __launch_bounds__(WAVE) void attention_general_kernel(
         const int j = lane + i * WAVE;
         if (j < vd) {
             if (all_v) o_wide[j] = acc[i] * inv;
+            else if (out_f32) ((float*)out)[((long long)t * H + head) * vd + j] = acc[i] * inv;
             else o[j] = from_f32<T>(acc[i] * inv);
         }
     }
@@ -131,18 +143,49 @@ TUFF_EXPORT int tuff_attention_general(const void* q, const void* k_cache, const
                                        const int* block_table, int max_blocks, const int* req_of_token,
                                        const int* positions, int n_tokens, int H, int Hkv, int hd, int vd, int page_size,
                                        int window, float scale, const float* sinks, const float* slopes, int v_in_k,
-                                       const float* log_r1, const float* log_r2, int all_v, hipStream_t stream) {
+                                       const float* log_r1, const float* log_r2, int all_v, int keep_first, int maps, int out_f32,
+                                       hipStream_t stream) {
     if (n_tokens <= 0) return 0;
+    if (maps < 1 || hd % maps || H % maps || keep_first < 0 || (out_f32 && all_v)) return -2;
     const int widest = max(hd, vd);
     if (widest > MAX_PER_LANE_WIDE * WAVE || vd <= 0 || Hkv <= 0 || H % Hkv != 0 || (v_in_k && vd > hd)) return -2;
     if ((log_r1 == nullptr) != (log_r2 == nullptr) || (all_v && v_in_k) || H > 65535 || Hkv > 65535) return -2;
     dim3 grid(n_tokens, H, all_v ? Hkv : 1), block(WAVE);
 #define LAUNCH(T, PL) hipLaunchKernelGGL((attention_general_kernel<T, PL>), grid, block, 0, stream, (const T*)q, (const T*)k_cache, \
         (const T*)v_cache, (T*)out, block_table, max_blocks, req_of_token, positions, H, Hkv, hd, vd, page_size, window, scale, \
-        sinks, slopes, v_in_k, log_r1, log_r2, all_v)
+        sinks, slopes, v_in_k, log_r1, log_r2, all_v, keep_first, maps, out_f32)
     if (widest <= 4 * WAVE) { if (dt == DT_F32) LAUNCH(float, 4); else LAUNCH(bf16_t, 4); }
     else { if (dt == DT_F32) LAUNCH(float, MAX_PER_LANE_WIDE); else LAUNCH(bf16_t, MAX_PER_LANE_WIDE); }
 #undef LAUNCH
+    return launch_status();
+}
+
+// Differential attention: a head's two maps a1, a2 (o float32 [T][2 H][vd], a head's maps side by side) become
+//   v = a1 - lambda * a2;   out[t][h] = v / sqrt(mean(v^2) + eps) * coef
+// A wave a (token, head); the row's sum of squares is a lane's channels in ascending order, then the wave's butterfly.
+namespace {
+template <typename T>
+__global__ __launch_bounds__(WAVE) void diff_combine_kernel(const float* __restrict__ o, T* __restrict__ out, int vd, float lambda,
+                                                            float eps, float coef) {
+    const long long row = blockIdx.x;
+    const float* a = o + row * 2 * vd;
+    float ss = 0.f;
+    for (int j = threadIdx.x; j < vd; j += WAVE) {
+        const float v = fmaf(-lambda, a[vd + j], a[j]);
+        ss = fmaf(v, v, ss);
+    }
+    const float inv = coef / sqrtf(wave_sum(ss) / (float)vd + eps);
+    for (int j = threadIdx.x; j < vd; j += WAVE) out[row * vd + j] = from_f32<T>(fmaf(-lambda, a[vd + j], a[j]) * inv);
+}
+}  // namespace
+
+TUFF_EXPORT int tuff_diff_combine(const float* o, void* out, int dt, int n_tokens, int H, int vd, float lambda, float eps, float coef,
+                                  hipStream_t stream) {
+    if (n_tokens <= 0) return 0;
+    const long long rows = (long long)n_tokens * H;
+    if (H <= 0 || vd <= 0 || rows > 0x7fffffffll) return -2;
+    if (dt == DT_F32) hipLaunchKernelGGL(diff_combine_kernel<float>, dim3((unsigned)rows), dim3(WAVE), 0, stream, o, (float*)out, vd, lambda, eps, coef);
+    else hipLaunchKernelGGL(diff_combine_kernel<bf16_t>, dim3((unsigned)rows), dim3(WAVE), 0, stream, o, (bf16_t*)out, vd, lambda, eps, coef);
     return launch_status();
 }
 

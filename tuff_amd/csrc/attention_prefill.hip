@@ -30,7 +30,13 @@
 // what the rounding left, in two products); and every query head's weights applied to the values of every kv
 // head (all_v: the grid's second axis is the kv head whose values are read, the sums are written in float32
 // as [token][head][kv head][vd]), from which a following kernel forms heads whose weights are mixtures of
-// the heads' softmax weights.
+// the heads' softmax weights.  A window may keep the sequence's first keys: the steps that hold them and lie before the
+// window's come first, and what a step hides is decided key by key.
+//
+// Differential attention (MAPS 2): a cached key row holds two keys side by side and a head has two softmax maps over the
+// same values.  A column is then a head of a token, and its two maps are the two column blocks of a wave: either meets
+// its own half of the key rows out of LDS, both meet the same values, and since both sums of a head end in the same
+// lanes, the epilogue takes the second map off the first, norms the head over its channels and writes the head once.
 #include "common.h"
 #include <math.h>
 
@@ -57,10 +63,12 @@ struct WideArgs {
     const float* log_r2;        // [H]
     int all_v;
     float* out_wide;            // all_v: float32 [token][head][kv head][vd]
+    int keep_first;             // with a window: keys before it are seen whatever the distance
+    float lambda, eps, coef;    // MAPS 2: v = a1 - lambda * a2, v / sqrt(mean(v^2) + eps) * coef
 };
 
-// HDP, VDP: the channels of a key and of a value in the tiles, multiples of 32.
-template <int HDP, int NBW, int AHEAD, bool EX, int VDP>
+// HDP, VDP: the channels of a key row and of a value in the tiles, multiples of 32 (a map's share of a key row too).
+template <int HDP, int NBW, int AHEAD, bool EX, int VDP, int MAPS>
 __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     bf16_t* __restrict__ out, const int* __restrict__ block_table, int max_blocks,
@@ -68,14 +76,16 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     int H, int Hkv, int hd, int page_size, int window, float scale_log2e,
     int seg_keys, float* __restrict__ ws_o, float* __restrict__ ws_ml, const float* __restrict__ sinks,
     const float* __restrict__ slopes, WideArgs wide) {
-    constexpr int KC = HDP / 32;          // 32-wide chunks of the head dimension
+    static_assert(MAPS == 1 || (MAPS == 2 && EX && NBW == 2), "two maps are the two column blocks of a wave of the wide form");
+    constexpr int HM = HDP / MAPS;        // channels of a map's key in the tiles
+    constexpr int KC = HM / 32;           // 32-wide chunks of a key
     constexpr int DB = VDP / 16;          // 16-wide blocks of output channels
     constexpr int HC = HDP / 8;           // 16-byte chunks of a K row
     constexpr int KROW = HDP + 8;         // bf16 a K row in LDS (padded like V^T rows)
     constexpr int KBUF = STEP * KROW, VBUF = VDP * VROW;
     constexpr int KPT = STEP * HC / NT;   // 16-byte pieces of K a thread copies a step
     constexpr int VPT = VDP * 8 / NT;     // and of V^T
-    constexpr int CB = 4 * NBW * 16;      // columns of a workgroup
+    constexpr int CB = 4 * NBW * 16 / MAPS;      // columns of a workgroup
     extern __shared__ __attribute__((aligned(16))) bf16_t lds[];
     bf16_t* Ks = lds;                     // [2][KBUF]
     bf16_t* Vs = lds + 2 * KBUF;          // [2][VBUF]
@@ -99,6 +109,8 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     const int last_col = min(ncols, col0 + CB) - 1;
     const int pos_max = pos0 + last_col / G;
     const int lo_min = window > 0 ? max(0, pos0 + col0 / G - window + 1) : 0;
+    const int keep = EX ? wide.keep_first : 0;
+    const int qd = hd / MAPS;              // channels of a query
     // gridDim.z > 1: the keys are cut into segments of seg_keys (a multiple of STEP), a workgroup a
     // segment; it leaves what it has summed, unnormalised, with its reference exponent and sum in
     // the work space, for the kernel that merges the partitions of single-token steps.
@@ -106,10 +118,13 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     const int seg_begin = n_segs > 1 ? seg * seg_keys : 0;
     const int key_last = n_segs > 1 ? min(pos_max, seg_begin + seg_keys - 1) : pos_max;
     const int key_start = max(lo_min / STEP * STEP, seg_begin);
-    const int nsteps = key_last >= key_start ? (key_last - key_start) / STEP + 1 : 0;
+    // the steps that hold first keys to keep and lie before the window's (the wide form is not cut into segments)
+    const int kept_steps = EX ? min((keep + STEP - 1) / STEP, key_start / STEP) : 0;
+    const int nsteps = key_last >= key_start ? (key_last - key_start) / STEP + 1 + kept_steps : 0;
+    auto key_of_step = [&](int s) { return EX && s < kept_steps ? s * STEP : key_start + (s - kept_steps) * STEP; };
 
     // ---- this wave's columns
-    const int wcol0 = col0 + wave * NBW * 16;
+    const int wcol0 = col0 + wave * NBW * 16 / MAPS;
     int pos_c[NBW], lo_c[NBW];
     float slope_c[NBW];                    // the head's distance slope, in base-2 exponents; 0: none
     float r1_c[NBW], r2_c[NBW];            // the head's logarithmic penalty: r1 * log2(1 + r2 * distance) in base-2 exponents
@@ -118,7 +133,8 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     int wave_pos_max = -1, wave_pos_min = 0x7fffffff, wave_lo_max = 0;
 #pragma unroll
     for (int nb = 0; nb < NBW; ++nb) {
-        const int c = wcol0 + nb * 16 + n16;
+        const int cb = MAPS == 2 ? 0 : nb * 16;        // (two maps: both blocks hold the same columns)
+        const int c = wcol0 + cb + n16;
         const bool valid = c < ncols;
         const int tok = t0 + (valid ? c / G : 0);
         const int head = kvh * G + (valid ? c % G : 0);
@@ -132,10 +148,10 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
         for (int kc = 0; kc < KC; ++kc) {
             const int k = kc * 32 + g * 8;
             bf16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
-            qf[nb][kc] = (valid && k < hd) ? *(const bf16x8*)(q + qrow[nb] * hd + k) : z;
+            qf[nb][kc] = (valid && k < qd) ? *(const bf16x8*)(q + (MAPS == 2 ? 2 * qrow[nb] + nb : qrow[nb]) * qd + k) : z;
         }
         // wave-wide: the range of positions of its columns (first and last column of the wave)
-        const int cf = wcol0 + nb * 16, cl = min(ncols - 1, wcol0 + nb * 16 + 15);
+        const int cf = wcol0 + cb, cl = min(ncols - 1, wcol0 + cb + 15);
         if (cf < ncols) {
             wave_pos_max = max(wave_pos_max, pos0 + cl / G);
             wave_pos_min = min(wave_pos_min, pos0 + cf / G);
@@ -171,10 +187,9 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
         return;
     }
 
-    // ---- page numbers: lane i holds the page of granule (16 keys) gran_base + i; 64 granules = 16 steps
-    const int gran0 = key_start / 16;
+    // ---- page numbers: lane i holds the page of granule (16 keys) i of sixteen steps, four a step
     auto pages_of = [&](int batch) {
-        const long long idx = ((long long)(gran0 + batch * 64 + lane) * 16) / page_size;
+        const long long idx = (long long)(key_of_step(batch * 16 + lane / 4) + 16 * (lane % 4)) / page_size;
         return idx < max_blocks ? table[idx] : -1;
     };
     int pages_cur = pages_of(0), pages_next = pages_of(1);
@@ -195,8 +210,9 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
         const int id = tid + i * NT, key = id / HC, c = id % HC;
         k_gran[i] = __builtin_amdgcn_readfirstlane(key / 16);
         k_key[i] = key;
-        k_off[i] = (key % 16) * hd + c * 8;
-        k_ok[i] = c * 8 < hd;
+        const int cm = c % (HM / 8);                    // (a map's part of the row lies at its own place in the tile)
+        k_off[i] = (key % 16) * hd + c / (HM / 8) * qd + cm * 8;
+        k_ok[i] = cm * 8 < qd;
         k_lds[i] = k_row_of_key(key) * KROW + c * 8;
     }
 #pragma unroll
@@ -208,15 +224,16 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
         v_ok[i] = dim < vd;
         v_lds[i] = dim * VROW + c8 * 8;
     }
-    const bool whole_rows = hd == HDP && vd == VDP;
+    const bool whole_rows = qd == HM && vd == VDP;
     const unsigned page_stride = (unsigned)(Hkv * page_size * hd);       // elements of a page in the key cache (the host checks that it fits)
     const unsigned head_off = (unsigned)(kvh * page_size * hd);          // this kv head's share of it
     const unsigned page_stride_v = (unsigned)(Hkv * page_size * vd);     // the same of the value cache
     const unsigned head_off_v = (unsigned)(vh * page_size * vd);
     const int ps_mask = (page_size & (page_size - 1)) == 0 ? page_size - 1 : 0;   // a power of two: offsets wrap by a mask
-    int ld_off = key_start % page_size;                 // offset in its page of the first key of the next step to load
+    int ld_off = key_of_step(0) % page_size;            // offset in its page of the first key of the next step to load
     auto load_step = [&](int set, int s, int pages) {   // step s of the block -> register set; zeros beyond pos_max
-        const int key0 = key_start + s * STEP;
+        const int key0 = key_of_step(s);
+        if (EX && s == kept_steps && kept_steps > 0) ld_off = key_start % page_size;      // from the first keys to the window's
         const int gslot0 = (s % 16) * 4;                // granule of the step's first key within `pages`
         // per piece, the same for the lanes of a wave: where its granule's rows start (-1: no such page)
         auto granule = [&](int g4, long long& base, int& go, bool values) {
@@ -299,10 +316,13 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
 #pragma unroll
             for (int nb = 0; nb < NBW; ++nb) sc.v[kb][nb] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int kc = 0; kc < KC; ++kc) {
+            for (int kc = 0; kc < KC * MAPS; ++kc) {
                 const bf16x8 kf = *(const bf16x8*)(Kb + kb * 16 * KROW + kc * 32);
+                if (MAPS == 2) sc.v[kb][kc / KC] = mfma32(kf, qf[kc / KC][kc % KC], sc.v[kb][kc / KC]);
+                else {
 #pragma unroll
-                for (int nb = 0; nb < NBW; ++nb) sc.v[kb][nb] = mfma32(kf, qf[nb][kc], sc.v[kb][nb]);
+                    for (int nb = 0; nb < NBW; ++nb) sc.v[kb][nb] = mfma32(kf, qf[nb][kc], sc.v[kb][nb]);
+                }
             }
         }
         return sc;
@@ -355,7 +375,7 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
 #pragma unroll
                     for (int e = 0; e < 4; ++e) {
                         const int key = key0 + 32 * sub + 8 * g + 4 * kb + e;
-                        const bool v = open || ((sub ? live1 : live0) && key <= pos_c[nb] && key >= lo_c[nb]);
+                        const bool v = open || ((sub ? live1 : live0) && key <= pos_c[nb] && (key >= lo_c[nb] || (EX && key < keep)));
                         ok[sub][kb * 4 + e] = v;
                         mx = fmaxf(mx, v ? sc[sub].v[kb][nb][e] : -INFINITY);
                     }
@@ -422,15 +442,15 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
             const int s = s0 + u;
             if (s >= nsteps) break;
             const int buf = s & 1;
-            const int key0 = key_start + s * STEP;
+            const int key0 = key_of_step(s);
             const int ls = s + AHEAD;                   // the step whose loads start now
             if (ls % 16 == 0) pages_cur = pages_next;
             if (ls % 16 == 1) pages_next = pages_of(ls / 16 + 1);
             load_step(u, ls, pages_cur);
             const int lo_any = window > 0 ? max(0, wave_pos_min - window + 1) : 0;
-            const bool live0 = key0 <= wave_pos_max && key0 + 31 >= lo_any;
-            const bool live1 = key0 + 32 <= wave_pos_max && key0 + 63 >= lo_any;
-            if (key0 + 63 <= wave_pos_min && key0 >= wave_lo_max) whole_step(buf, key0, true, true, std::true_type());
+            const bool live0 = key0 <= wave_pos_max && (key0 + 31 >= lo_any || (EX && key0 < keep));
+            const bool live1 = key0 + 32 <= wave_pos_max && (key0 + 63 >= lo_any || (EX && key0 + 32 < keep));
+            if (key0 + 63 <= wave_pos_min && (key0 >= wave_lo_max || (EX && key0 + 63 < keep))) whole_step(buf, key0, true, true, std::true_type());
             else if (live0 || live1) whole_step(buf, key0, live0, live1, std::false_type());
             store_step((u + 1) % AHEAD, buf ^ 1);
             __syncthreads();
@@ -438,6 +458,33 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     }
 
     // ---- normalise and write
+    if constexpr (MAPS == 2) {
+        // lane (column n16, group g) holds channels 16 db + 4 g .. + 3 of both maps of its head
+        const float inv0 = 1.0f / __shfl(l_acc[0][0], n16, WAVE), inv1 = wide.lambda / __shfl(l_acc[1][0], n16, WAVE);
+        float ss = 0.f;
+#pragma unroll
+        for (int db = 0; db < DB; ++db)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {                      // (channels beyond vd are zeros in both)
+                const float v = fmaf(-inv1, o[db][1][e], o[db][0][e] * inv0);
+                o[db][0][e] = v;
+                ss = fmaf(v, v, ss);
+            }
+        ss += __shfl_xor(ss, 16, WAVE);
+        ss += __shfl_xor(ss, 32, WAVE);
+        if (qrow[0] < 0) return;
+        const float by = wide.coef / sqrtf(ss / (float)vd + wide.eps);
+#pragma unroll
+        for (int db = 0; db < DB; ++db) {
+            const int dim = db * 16 + 4 * g;
+            if (dim < vd) {
+                const f32x4 v = o[db][0];
+                bf16x4 w = {(bf16_t)(v[0] * by), (bf16_t)(v[1] * by), (bf16_t)(v[2] * by), (bf16_t)(v[3] * by)};
+                *(bf16x4*)(out + qrow[0] * vd + dim) = w;
+            }
+        }
+        return;
+    }
 #pragma unroll
     for (int nb = 0; nb < NBW; ++nb) {
         const float l = __shfl(l_acc[nb][0], n16, WAVE);       // from the lane of group 0 that holds the column's sum
@@ -485,12 +532,12 @@ __global__ __launch_bounds__(NT) void attn_prefill_kernel(
     }
 }
 
-template <int HDP, int NBW, int AHEAD, bool EX = false, int VDP = HDP>
+template <int HDP, int NBW, int AHEAD, bool EX = false, int VDP = HDP, int MAPS = 1>
 int launch(dim3 grid, hipStream_t stream, const bf16_t* q, const bf16_t* kc, const bf16_t* vc, bf16_t* out,
            const int* bt, int max_blocks, const int2* blk, const int4* req_info,
            int H, int Hkv, int hd, int ps, int window, float scale_log2e, int seg_keys, float* ws_o, float* ws_ml,
-           const float* sinks, const float* slopes, WideArgs wide = WideArgs{0, nullptr, nullptr, 0, nullptr}) {
-    auto kern = attn_prefill_kernel<HDP, NBW, AHEAD, EX, VDP>;
+           const float* sinks, const float* slopes, WideArgs wide = WideArgs{0, nullptr, nullptr, 0, nullptr, 0, 0.f, 0.f, 0.f}) {
+    auto kern = attn_prefill_kernel<HDP, NBW, AHEAD, EX, VDP, MAPS>;
     constexpr int lds = 2 * (STEP * (HDP + 8) + VDP * VROW) * 2;
     static bool set = false;
     if (!set) {
@@ -565,19 +612,20 @@ TUFF_EXPORT int tuff_attention_prefill(const void* q, const void* k_cache, const
 // The wide form: values vd channels wide (V [page][kv_head][vd][offset]), weights that keep float32's precision,
 // log_r1, log_r2 (float32 [H], or both null): r1[h] * ln(1 + r2[h] * (position - key)) is taken off head h's scaled
 // scores.  all_v: every head's weights on every kv head's values, out is then float32 [tokens][H][Hkv][vd]; else out
-// is bfloat16 [tokens][H][vd].  Keys are not cut into segments.
+// is bfloat16 [tokens][H][vd].  Keys are not cut into segments.  keep_first: with a window, keys before it are seen whatever
+// the distance.
 TUFF_EXPORT int tuff_attention_prefill_wide(const void* q, const void* k_cache, const void* v_cache, void* out,
                                             const int* block_table, int max_blocks, const int* blk, int n_qblocks,
                                             const int* req_info, int H, int Hkv, int hd, int vd, int page_size, int window,
                                             float scale, const float* sinks, const float* slopes, const float* log_r1,
-                                            const float* log_r2, int all_v, hipStream_t stream) {
+                                            const float* log_r2, int all_v, int keep_first, hipStream_t stream) {
     if (n_qblocks <= 0) return 0;
     if (hd > 256 || hd % 8 != 0 || vd > 256 || vd <= 0 || vd % 8 != 0 || page_size % 16 != 0 || Hkv <= 0 || H % Hkv != 0) return -2;
-    if (Hkv > 65535 || !(scale > 0.f) || (log_r1 == nullptr) != (log_r2 == nullptr)) return -2;
+    if (Hkv > 65535 || !(scale > 0.f) || (log_r1 == nullptr) != (log_r2 == nullptr) || keep_first < 0) return -2;
     if ((long long)Hkv * page_size * max(hd, vd) > 0x7fffffffll || (long long)n_qblocks * Hkv > 0x7fffffffll) return -2;
     dim3 grid(n_qblocks * Hkv, all_v ? Hkv : 1, 1);
     const float sl = scale * 1.4426950408889634f;
-    const WideArgs wide{vd, log_r1, log_r2, all_v, all_v ? (float*)out : nullptr};
+    const WideArgs wide{vd, log_r1, log_r2, all_v, all_v ? (float*)out : nullptr, window > 0 ? keep_first : 0, 0.f, 0.f, 0.f};
     const int widest = max(hd, vd);
 #define GO(HDP, NBW, AHEAD, VDP) return launch<HDP, NBW, AHEAD, true, VDP>(grid, stream, (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, \
         (bf16_t*)out, block_table, max_blocks, (const int2*)blk, (const int4*)req_info, H, Hkv, hd, page_size, window, sl, 0, nullptr, \
@@ -592,5 +640,34 @@ TUFF_EXPORT int tuff_attention_prefill_wide(const void* q, const void* k_cache, 
     else if (widest <= 224) GO(224, 2, 1, 224);
     else if (vd <= 192) GO(256, 2, 1, 192);
     else GO(256, 2, 1, 256);
+#undef GO
+}
+
+// Differential attention: K [page][kv_head][offset][2 dim], two keys a row; q [tokens][heads][2][dim]; every head's two
+// softmax maps over the values of its kv head, combined: v = a1 - lambda * a2, out bfloat16 [tokens][heads][vd] =
+// v / sqrt(mean(v^2) + eps) * coef.  Weights keep float32's precision.  A block of the list holds
+// tuff_attention_prefill_diff_block_columns() columns, a column a head of a token.
+TUFF_EXPORT int tuff_attention_prefill_diff_block_columns(void) { return 64; }
+
+TUFF_EXPORT int tuff_attention_prefill_diff(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                            const int* block_table, int max_blocks, const int* blk, int n_qblocks,
+                                            const int* req_info, int heads, int Hkv, int dim, int vd, int page_size, int window,
+                                            int keep_first, float scale, float lambda, float eps, float coef, hipStream_t stream) {
+    if (n_qblocks <= 0) return 0;
+    if (dim > 128 || dim < 8 || dim % 8 != 0 || vd > 256 || vd <= 0 || vd % 8 != 0 || page_size % 16 != 0 || Hkv <= 0 || heads % Hkv != 0) return -2;
+    if (Hkv > 65535 || !(scale > 0.f) || keep_first < 0) return -2;
+    const int hd = 2 * dim;
+    if ((long long)Hkv * page_size * max(hd, vd) > 0x7fffffffll || (long long)n_qblocks * Hkv > 0x7fffffffll) return -2;
+    dim3 grid(n_qblocks * Hkv, 1, 1);
+    const float sl = scale * 1.4426950408889634f;
+    const WideArgs wide{vd, nullptr, nullptr, 0, nullptr, window > 0 ? keep_first : 0, lambda, eps, coef};
+#define GO(HDP, AHEAD, VDP) return launch<HDP, 2, AHEAD, true, VDP, 2>(grid, stream, (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, \
+        (bf16_t*)out, block_table, max_blocks, (const int2*)blk, (const int4*)req_info, heads, Hkv, hd, page_size, window, sl, 0, nullptr, \
+        nullptr, nullptr, nullptr, wide)
+    if (dim <= 32) { if (vd <= 64) GO(64, 2, 64); else if (vd <= 128) GO(64, 2, 128); else GO(64, 1, 256); }
+    if (dim <= 64) { if (vd <= 64) GO(128, 2, 64); else if (vd <= 128) GO(128, 2, 128); else GO(128, 1, 256); }
+    if (dim <= 96) { if (vd <= 128) GO(192, 1, 128); else if (vd <= 192) GO(192, 1, 192); else GO(192, 1, 256); }
+    if (vd <= 128) GO(256, 1, 128);
+    GO(256, 1, 256);
 #undef GO
 }

@@ -12,7 +12,13 @@
 // ascending order and lets a head's sink (a logit without key or value) into the denominator.
 //
 // With a window the parts of a token are counted from the first one its window touches, so that a launch has as many
-// parts as a window can touch, whatever the context.
+// parts as a window can touch, whatever the context.  A window may keep the sequence's first keys (keep_first): the parts
+// that hold them and lie before the window's come first.
+//
+// A cached key row may hold `maps` keys side by side (differential attention: two softmax maps over one kv head's values).
+// H then counts maps: column c of a token meets part c % maps of the row with its hd / maps query channels, zeros stand in
+// its operand for the other parts, so the row is read once for all maps.  The merge then combines a head's two maps a1, a2:
+// v = a1 - lambda * a2, v / sqrt(mean(v^2) + eps) * coef.
 //
 // Cache layout: K [page][kv_head][offset][hd], V [page][kv_head][vd][offset]; page sizes are multiples of 16, hd and vd
 // multiples of 8 up to 256.
@@ -27,6 +33,16 @@ constexpr int XCDS = 8;
 
 __device__ __forceinline__ f32x4 mfma32(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
 
+// The part of keys that a token's slot stands for: the parts of first keys that lie before its window's (lo: the window's
+// first key), then the window's.
+__device__ __forceinline__ int kept_parts(int lo, int keep_first, int part_keys) {
+    return min((keep_first + part_keys - 1) / part_keys, lo / part_keys);
+}
+__device__ __forceinline__ int part_of_slot(int slot, int lo, int keep_first, int part_keys) {
+    const int kept = kept_parts(lo, keep_first, part_keys);
+    return slot < kept ? slot : lo / part_keys + (slot - kept);
+}
+
 // KC: 32-wide pieces of the key size; DBW: 16-wide blocks of value channels a wave.
 template <int KC, int DBW>
 __global__ __launch_bounds__(NT) void single_part_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache,
@@ -34,7 +50,8 @@ __global__ __launch_bounds__(NT) void single_part_kernel(const bf16_t* __restric
                                                          float* __restrict__ ws_ml, const int* __restrict__ block_table, int max_blocks,
                                                          const int* __restrict__ req_of_token, const int* __restrict__ positions,
                                                          int n_tokens, int H, int Hkv, int hd, int vd, int page_size, int window, float scale,
-                                                         const float* __restrict__ slopes, int part_keys, int n_slots, int chunks) {
+                                                         const float* __restrict__ slopes, int part_keys, int n_slots, int chunks,
+                                                         int keep_first, int maps) {
     __shared__ float red[WAVES][16];
     __shared__ __attribute__((aligned(16))) bf16_t p_hi[16 * PSTRIDE], p_lo[16 * PSTRIDE];
     // workgroups that read the same keys (the chunks of heads of one part) follow each other on one XCD
@@ -45,18 +62,19 @@ __global__ __launch_bounds__(NT) void single_part_kernel(const bf16_t* __restric
     const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, n16 = lane % 16, g = lane / 16;
     const int pos = positions[t];
     const int lo = window > 0 ? max(0, pos - window + 1) : 0;
-    const int key_begin = (lo / part_keys + slot) * part_keys;
+    const int key_begin = part_of_slot(slot, lo, keep_first, part_keys) * part_keys;
     if (key_begin > pos) return;
     const int key_end = min(key_begin + part_keys, pos + 1);
     const int* table = block_table + (long long)req_of_token[t] * max_blocks;
     const bf16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
 
     bf16x8 qf[KC];
-    const bf16_t* qrow = q + ((long long)t * H + head0 + min(n16, cols - 1)) * hd;
+    const int qd = hd / maps, q_from = ((head0 + min(n16, cols - 1)) % maps) * qd;       // the column's part of the key row
+    const bf16_t* qrow = q + ((long long)t * H + head0 + min(n16, cols - 1)) * qd;
 #pragma unroll
     for (int kc = 0; kc < KC; ++kc) {
-        const int k = kc * 32 + g * 8;
-        qf[kc] = (n16 < cols && k < hd) ? *(const bf16x8*)(qrow + k) : zero;
+        const int k = kc * 32 + g * 8 - q_from;
+        qf[kc] = (n16 < cols && k >= 0 && k < qd) ? *(const bf16x8*)(qrow + k) : zero;
     }
     const float slope = slopes ? slopes[head0 + min(n16, cols - 1)] : 0.f;
 
@@ -66,18 +84,18 @@ __global__ __launch_bounds__(NT) void single_part_kernel(const bf16_t* __restric
     for (int db = 0; db < DBW; ++db) o[db] = f32x4{0.f, 0.f, 0.f, 0.f};
 
     for (int key0 = key_begin; key0 < key_end; key0 += BLOCK) {
-        if (key0 + BLOCK <= lo) continue;                     // (uniform) the window has passed the block
+        if (key0 + BLOCK <= lo && key0 >= keep_first) continue;       // (uniform) the window has passed the block
         // the block's eight sixteens of keys lie in a page each: lane i fetches the i-th one's page number
         int my_page = 0;
         {
             const int k = key0 + 16 * (lane % 8);
-            if (k <= pos && k + 15 >= lo) my_page = table[k / page_size];
+            if (k <= pos && (k + 15 >= lo || k < keep_first)) my_page = table[k / page_size];
         }
         bf16x8 kf[2][KC];
 #pragma unroll
         for (int h = 0; h < 2; ++h) {
             const int k16 = key0 + 32 * wave + 16 * h;
-            const bool live = k16 <= pos && k16 + 15 >= lo;
+            const bool live = k16 <= pos && (k16 + 15 >= lo || k16 < keep_first);
             const long long page = __shfl(my_page, 2 * wave + h, WAVE);
             const bf16_t* row = k_cache + ((page * Hkv + kvh) * page_size + k16 % page_size + n16) * hd;
 #pragma unroll
@@ -90,7 +108,7 @@ __global__ __launch_bounds__(NT) void single_part_kernel(const bf16_t* __restric
 #pragma unroll
         for (int ks = 0; ks < 4; ++ks) {
             const int k8 = key0 + 32 * ks + 8 * g;
-            const bool live = k8 <= pos && k8 + 7 >= lo;
+            const bool live = k8 <= pos && (k8 + 7 >= lo || k8 < keep_first);
             const long long page = __shfl(my_page, 2 * ks + g / 2, WAVE);
             const bf16_t* at = v_cache + (page * Hkv + kvh) * (long long)vd * page_size + k8 % page_size;
 #pragma unroll
@@ -110,7 +128,7 @@ __global__ __launch_bounds__(NT) void single_part_kernel(const bf16_t* __restric
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const int key = key0 + 32 * wave + 16 * h + 4 * g + e;
-                v[h][e] = (key >= lo && key <= pos) ? fmaf(s[e], scale, -slope * (float)(pos - key)) : -INFINITY;
+                v[h][e] = ((key >= lo || key < keep_first) && key <= pos) ? fmaf(s[e], scale, -slope * (float)(pos - key)) : -INFINITY;
                 mx = fmaxf(mx, v[h][e]);
             }
         }
@@ -188,12 +206,12 @@ constexpr int MAX_PART = 1024;             // keys; a plan's parts are longer on
 template <typename T>
 __global__ __launch_bounds__(256) void single_merge_kernel(const float* __restrict__ ws_o, const float* __restrict__ ws_ml, T* __restrict__ out,
                                                            const int* __restrict__ positions, const float* __restrict__ sinks, int H, int vd,
-                                                           int window, int part_keys, int n_slots) {
+                                                           int window, int part_keys, int n_slots, int keep_first) {
     const long long row = blockIdx.x;
     const int lane = threadIdx.x % WAVE, ch = threadIdx.x;
     const int pos = positions[row / H];
     const int lo = window > 0 ? max(0, pos - window + 1) : 0;
-    const int parts = min(n_slots, pos / part_keys - lo / part_keys + 1);
+    const int parts = min(n_slots, kept_parts(lo, keep_first, part_keys) + pos / part_keys - lo / part_keys + 1);
     float m = -INFINITY, l = 0.f;
     if (lane < parts) {
         const float2 ml = *(const float2*)(ws_ml + (row * n_slots + lane) * 2);
@@ -217,38 +235,94 @@ __global__ __launch_bounds__(256) void single_merge_kernel(const float* __restri
     }
     if (ch < vd) out[row * vd + ch] = from_f32<T>(acc * inv);
 }
+
+// A workgroup a (token, head) of differential attention: the parts of both maps merged as above, then combined and normed
+// over the head's channels.
+template <typename T>
+__global__ __launch_bounds__(256) void single_merge_diff_kernel(const float* __restrict__ ws_o, const float* __restrict__ ws_ml, T* __restrict__ out,
+                                                                const int* __restrict__ positions, int heads, int vd, int window, int part_keys,
+                                                                int n_slots, int keep_first, float lambda, float eps, float coef) {
+    __shared__ float scratch[4];
+    const long long row = blockIdx.x;
+    const int lane = threadIdx.x % WAVE, ch = threadIdx.x;
+    const int pos = positions[row / heads];
+    const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+    const int parts = min(n_slots, kept_parts(lo, keep_first, part_keys) + pos / part_keys - lo / part_keys + 1);
+    float w[2], inv[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        float m = -INFINITY, l = 0.f;
+        if (lane < parts) {
+            const float2 ml = *(const float2*)(ws_ml + ((2 * row + i) * n_slots + lane) * 2);
+            m = ml.x;
+            l = ml.y;
+        }
+        const float M = wave_max(m);
+        w[i] = lane < parts ? __expf(m - M) : 0.f;
+        inv[i] = 1.0f / wave_sum(w[i] * l);
+    }
+    const float* o = ws_o + 2 * row * n_slots * vd + ch;
+    const long long other = (long long)n_slots * vd;           // from the first map's parts to the second's
+    float acc[2] = {0.f, 0.f};
+    for (int p0 = 0; p0 < parts; p0 += 4) {
+        float x[2][4];
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+            for (int u = 0; u < 4; ++u) x[i][u] = (p0 + u < parts && ch < vd) ? o[i * other + (long long)(p0 + u) * vd] : 0.f;
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+            for (int u = 0; u < 4; ++u) acc[i] = fmaf(__shfl(w[i], min(p0 + u, WAVE - 1), WAVE), x[i][u], acc[i]);
+    }
+    const float v = ch < vd ? fmaf(-lambda, acc[1] * inv[1], acc[0] * inv[0]) : 0.f;
+    // the row's sum of squares: the waves' butterflies, then the waves in order
+    const float ss = wave_sum(v * v);
+    if (lane == 0) scratch[threadIdx.x / WAVE] = ss;
+    __syncthreads();
+    float sum = 0.f;
+    for (int i = 0; i < (int)blockDim.x / WAVE; ++i) sum += scratch[i];
+    if (ch < vd) out[row * vd + ch] = from_f32<T>(v * (coef / sqrtf(sum / (float)vd + eps)));
+}
 }  // namespace
 
-// Parts a token's keys can touch with parts of part_keys keys: with a window as many as the window touches at any place.
-static int slots_of(int max_ctx_len, int window, int part_keys) {
+// Parts a token's keys can touch with parts of part_keys keys: with a window as many as the window touches at any place, and
+// those of the first keys that stay.
+static int slots_of(int max_ctx_len, int window, int part_keys, int keep_first) {
     const int all = ceil_div(max_ctx_len < 1 ? 1 : max_ctx_len, part_keys);
     if (window <= 0) return all;
-    const int touched = (int)(((long long)window + part_keys - 2) / part_keys) + 1;
-    return touched < all ? touched : all;
+    const long long touched = ((long long)window + part_keys - 2) / part_keys + 1 + ceil_div(keep_first, part_keys);
+    return touched < all ? (int)touched : all;
 }
 
 // How a launch is cut: *part_keys (a multiple of 128) and *n_slots parts a token, for work arrays ws_o float32
 // [n_tokens * H * n_slots * vd] and ws_ml float32 [n_tokens * H * n_slots * 2].  Parts of 128 keys while that leaves at most 2,048
 // workgroups, longer ones (up to 1,024 keys) beyond, and at most 64 of them.
-TUFF_EXPORT int tuff_attention_single_plan(int n_tokens, int H, int Hkv, int max_ctx_len, int window, int* part_keys, int* n_slots) {
-    if (n_tokens < 1 || Hkv < 1 || H < 1 || H % Hkv || !part_keys || !n_slots) return -2;
+TUFF_EXPORT int tuff_attention_single_plan(int n_tokens, int H, int Hkv, int max_ctx_len, int window, int keep_first, int* part_keys, int* n_slots) {
+    if (n_tokens < 1 || Hkv < 1 || H < 1 || H % Hkv || keep_first < 0 || !part_keys || !n_slots) return -2;
     const long long rows = (long long)n_tokens * Hkv * ceil_div(H / Hkv, 16);
     int pk = BLOCK;
-    while (pk < MAX_PART && rows * slots_of(max_ctx_len, window, pk) > 2048) pk += BLOCK;
-    while (slots_of(max_ctx_len, window, pk) > MAX_SLOTS) pk += BLOCK;
+    while (pk < MAX_PART && rows * slots_of(max_ctx_len, window, pk, keep_first) > 2048) pk += BLOCK;
+    while (slots_of(max_ctx_len, window, pk, keep_first) > MAX_SLOTS) pk += BLOCK;
     *part_keys = pk;
-    *n_slots = slots_of(max_ctx_len, window, pk);
+    *n_slots = slots_of(max_ctx_len, window, pk, keep_first);
     return 0;
 }
 
 // Row i of q [n_tokens][H * hd] and out [n_tokens][H * vd] is a token at positions[i] of request req_of_token[i], which sees
 // the cached keys up to itself (the last `window` of them, if positive); part_keys and n_slots from the plan for a
-// max_ctx_len that bounds every position + 1.  sinks, slopes: float32 [H] or null.
+// max_ctx_len that bounds every position + 1.  sinks, slopes: float32 [H] or null.  keep_first: with a window, keys before it
+// are seen whatever the distance.  maps 2: a key row holds two keys of hd / 2 channels, q is [n_tokens][H][hd / 2] with a
+// head's maps side by side (H counts maps, an even number a kv head), and out [n_tokens][H / 2 * vd] is what the merge makes of a
+// head's two maps with lambda, eps and coef (no sinks then).
 TUFF_EXPORT int tuff_attention_single(const void* q, const void* k_cache, const void* v_cache, void* out, int out_dt, float* ws_o, float* ws_ml,
                                       const int* block_table, int max_blocks, const int* req_of_token, const int* positions, int n_tokens,
                                       int H, int Hkv, int hd, int vd, int page_size, int window, float scale, const float* sinks,
-                                      const float* slopes, int part_keys, int n_slots, hipStream_t stream) {
+                                      const float* slopes, int part_keys, int n_slots, int keep_first, int maps, float lambda, float eps,
+                                      float coef, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
+    if (keep_first < 0 || maps < 1 || maps > 2 || (maps == 2 && (hd % 16 || (H / (Hkv < 1 ? 1 : Hkv)) % 2 || sinks))) return -2;
+    if (window <= 0) keep_first = 0;
     if (Hkv < 1 || H < 1 || H % Hkv || hd < 8 || hd > 256 || hd % 8 || vd < 8 || vd > 256 || vd % 8 || page_size < 16 || page_size % 16) return -2;
     if (part_keys < BLOCK || part_keys % BLOCK || n_slots < 1 || n_slots > MAX_SLOTS || max_blocks < 1) return -2;
     const int chunks = ceil_div(H / Hkv, 16);
@@ -257,14 +331,23 @@ TUFF_EXPORT int tuff_attention_single(const void* q, const void* k_cache, const 
     if (groups > 0x7fffffffll || (long long)n_tokens * H > 0x7fffffffll) return -2;
 #define GO(KC, DBW) hipLaunchKernelGGL((single_part_kernel<KC, DBW>), dim3((unsigned)groups), dim3(NT), 0, stream, (const bf16_t*)q, \
         (const bf16_t*)k_cache, (const bf16_t*)v_cache, ws_o, ws_ml, block_table, max_blocks, req_of_token, positions, n_tokens, H, Hkv, hd, \
-        vd, page_size, window, scale, slopes, part_keys, n_slots, chunks)
+        vd, page_size, window, scale, slopes, part_keys, n_slots, chunks, keep_first, maps)
     const int widest = hd > vd ? hd : vd;
     if (widest <= 64) GO(2, 1); else if (widest <= 128) GO(4, 2); else GO(8, 4);
 #undef GO
     const int rc = launch_status();
     if (rc) return rc;
-    const dim3 grid(n_tokens * H), block(ceil_div(vd, WAVE) * WAVE);
-    if (out_dt == DT_F32) hipLaunchKernelGGL(single_merge_kernel<float>, grid, block, 0, stream, ws_o, ws_ml, (float*)out, positions, sinks, H, vd, window, part_keys, n_slots);
-    else hipLaunchKernelGGL(single_merge_kernel<bf16_t>, grid, block, 0, stream, ws_o, ws_ml, (bf16_t*)out, positions, sinks, H, vd, window, part_keys, n_slots);
+    const dim3 block(ceil_div(vd, WAVE) * WAVE);
+    if (maps == 2) {
+        const dim3 rows(n_tokens * (H / 2));
+#define MERGE(T) hipLaunchKernelGGL(single_merge_diff_kernel<T>, rows, block, 0, stream, ws_o, ws_ml, (T*)out, positions, H / 2, vd, window, part_keys, \
+        n_slots, keep_first, lambda, eps, coef)
+        if (out_dt == DT_F32) MERGE(float); else MERGE(bf16_t);
+#undef MERGE
+        return launch_status();
+    }
+    const dim3 grid(n_tokens * H);
+    if (out_dt == DT_F32) hipLaunchKernelGGL(single_merge_kernel<float>, grid, block, 0, stream, ws_o, ws_ml, (float*)out, positions, sinks, H, vd, window, part_keys, n_slots, keep_first);
+    else hipLaunchKernelGGL(single_merge_kernel<bf16_t>, grid, block, 0, stream, ws_o, ws_ml, (bf16_t*)out, positions, sinks, H, vd, window, part_keys, n_slots, keep_first);
     return launch_status();
 }

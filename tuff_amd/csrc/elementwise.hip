@@ -6,24 +6,25 @@
 // ------------------------------------------------------------------ embedding
 // out[t, :] = table[tokens[t], :] * scale as float32.  Reference: one row gather per token
 // with no scale (src/lfm25_gpu.cu:725-741), which is scale = 1: the product with 1 is exact.
-template <typename T>
+template <typename T, typename TO>
 __global__ void embed_rows_kernel(const T* __restrict__ table, const int* __restrict__ tokens,
-                                  float* __restrict__ out, int d, float scale) {
+                                  TO* __restrict__ out, int d, float scale) {
     const int t = blockIdx.x;
     const long long row = tokens[t];
     const T* src = table + row * (long long)d;
-    float* dst = out + (long long)t * d;
-    for (int i = threadIdx.x; i < d; i += blockDim.x) dst[i] = to_f32(src[i]) * scale;
+    TO* dst = out + (long long)t * d;
+    for (int i = threadIdx.x; i < d; i += blockDim.x) dst[i] = from_f32<TO>(to_f32(src[i]) * scale);
 }
 
-TUFF_EXPORT int tuff_embed_rows(const void* table, int table_dt, const int* tokens, float* out,
+// out_dt: float32 (the residual stream), or the compute type for whoever reads the embedding itself.
+TUFF_EXPORT int tuff_embed_rows(const void* table, int table_dt, const int* tokens, void* out, int out_dt,
                                 int n_tokens, int d, float scale, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     dim3 grid(n_tokens), block(256);
-    if (table_dt == DT_F32)
-        hipLaunchKernelGGL(embed_rows_kernel<float>, grid, block, 0, stream, (const float*)table, tokens, out, d, scale);
-    else
-        hipLaunchKernelGGL(embed_rows_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)table, tokens, out, d, scale);
+#define LAUNCH(T, TO) hipLaunchKernelGGL((embed_rows_kernel<T, TO>), grid, block, 0, stream, (const T*)table, tokens, (TO*)out, d, scale)
+    if (table_dt == DT_F32) { if (out_dt == DT_F32) LAUNCH(float, float); else LAUNCH(float, bf16_t); }
+    else { if (out_dt == DT_F32) LAUNCH(bf16_t, float); else LAUNCH(bf16_t, bf16_t); }
+#undef LAUNCH
     return launch_status();
 }
 
@@ -359,6 +360,52 @@ TUFF_EXPORT int tuff_act_rows(const void* in, int in_dt, void* out, int out_dt, 
 #define LAUNCH(TI, TO) hipLaunchKernelGGL((act_rows_kernel<TI, TO>), grid, block, 0, stream, (const TI*)in, (TO*)out, n, N, kind, row_gate, gate_stride, gate_kind, col_bias, params)
     if (in_dt == DT_F32 && out_dt == DT_F32) LAUNCH(float, float);
     else if (in_dt == DT_F32) LAUNCH(float, bf16_t);
+    else if (out_dt == DT_F32) LAUNCH(bf16_t, float);
+    else LAUNCH(bf16_t, bf16_t);
+#undef LAUNCH
+    return launch_status();
+}
+
+// out[t, c] = f(in[t, c]) * table[tokens[t], col0 + c] for c < N, zeros for N <= c < Np: an activation times a vector looked
+// up by the token's id, rows as wide as the product that follows reads them.  VEC neighbouring columns a thread.
+template <typename TT, typename TO, int VEC>
+__global__ void act_lookup_kernel(const float* __restrict__ in, const TT* __restrict__ table, const int* __restrict__ tokens,
+                                  TO* __restrict__ out, long long n, int N, int Np, int kind, long long table_stride, int col0) {
+    const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= n) return;
+    const int per = Np / VEC;
+    const long long t = i / per;
+    const int c = (int)(i - t * per) * VEC;
+    const TT* row = table + tokens[t] * table_stride + col0;
+    typedef float in_v __attribute__((ext_vector_type(VEC)));
+    typedef TT tab_v __attribute__((ext_vector_type(VEC)));
+    typedef TO out_v __attribute__((ext_vector_type(VEC)));
+    out_v o;
+    if (c < N) {
+        const in_v z = *(const in_v*)(in + t * N + c);
+        const tab_v e = *(const tab_v*)(row + c);
+#pragma unroll
+        for (int k = 0; k < VEC; ++k) o[k] = from_f32<TO>(activation(z[k], kind) * to_f32((TT)e[k]));
+    } else {
+#pragma unroll
+        for (int k = 0; k < VEC; ++k) o[k] = from_f32<TO>(0.f);
+    }
+    *(out_v*)(out + t * Np + c) = o;
+}
+
+// table [*][table_stride] of type table_dt, tokens int32 [rows] (ids the caller has checked), out [rows][Np] of type out_dt.
+TUFF_EXPORT int tuff_act_lookup(const float* in, const void* table, int table_dt, const int* tokens, void* out, int out_dt, long long rows,
+                                int N, int Np, int kind, long long table_stride, int col0, hipStream_t stream) {
+    if (rows <= 0 || N <= 0) return 0;
+    if (Np < N || col0 < 0 || col0 + N > table_stride || kind == 7 || kind == 5) return -2;
+    const bool four = N % 4 == 0 && Np % 4 == 0 && col0 % 4 == 0 && table_stride % 4 == 0;
+    const long long n = rows * (four ? Np / 4 : Np);
+    const dim3 grid((unsigned)ceil_div_ll(n, 256)), block(256);
+#define LAUNCH(TT, TO) do { \
+    if (four) hipLaunchKernelGGL((act_lookup_kernel<TT, TO, 4>), grid, block, 0, stream, in, (const TT*)table, tokens, (TO*)out, n, N, Np, kind, table_stride, col0); \
+    else hipLaunchKernelGGL((act_lookup_kernel<TT, TO, 1>), grid, block, 0, stream, in, (const TT*)table, tokens, (TO*)out, n, N, Np, kind, table_stride, col0); } while (0)
+    if (table_dt == DT_F32 && out_dt == DT_F32) LAUNCH(float, float);
+    else if (table_dt == DT_F32) LAUNCH(float, bf16_t);
     else if (out_dt == DT_F32) LAUNCH(bf16_t, float);
     else LAUNCH(bf16_t, bf16_t);
 #undef LAUNCH

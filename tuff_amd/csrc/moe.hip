@@ -12,7 +12,11 @@
 // The router may have a bias: z = W h + b.  A limited choice (sigmoid weights): the choice runs on
 // c = sigmoid(z) + correction instead of z, and only inside the `keep` groups of neighbouring experts (of `groups`
 // equal ones) whose two largest c have the largest sum; the weights are the chosen experts' sigmoid(z), without the
-// correction, times a constant.  A (token, choice) pair is a
+// correction, times a constant.  A corrected choice (softmax weights): the choice runs on c = softmax over all outputs of the
+// router + correction; the weights are the chosen ones' softmax without the correction, divided by their sum (+ 1e-20).
+// The router may have more outputs than there are experts: a choice beyond the last expert is an identity expert, whose
+// output is the token's input itself; it is no row of the experts' products and joins when a token's rows are
+// added up.  A (token, choice) pair is a
 // row of the work arrays; the rows of a token are added into the residual stream in the order of
 // its choices, so the sum does not depend on what else is in the step.
 #include "common.h"
@@ -112,6 +116,45 @@ __device__ void choose_limited(const float* row, float* cs, int* ids, float* wts
     }
 }
 
+// The corrected choice of one token, by a whole wave (see the head of the file).  row: its N logits, cs: N floats of
+// scratch, both in LDS.  A lane holds every 64th output; sums and maxima meet in butterflies, ties go to the lower index.
+__device__ void choose_corrected(const float* row, float* cs, int* ids, float* wts, long long t, int N, int top, const float* corr) {
+    const int lane = threadIdx.x % WAVE;
+    float zmax = -INFINITY;
+    for (int e = lane; e < N; e += WAVE) zmax = fmaxf(zmax, row[e]);
+    zmax = wave_max(zmax);
+    float den = 0.f;
+    for (int e = lane; e < N; e += WAVE) den += expf(row[e] - zmax);
+    den = wave_sum(den);
+    for (int e = lane; e < N; e += WAVE) cs[e] = expf(row[e] - zmax) / den + (corr ? corr[e] : 0.f);
+    // (a lane reads back only what it wrote itself; a chosen output's place is taken out of the running)
+    float mine = 0.f, sum = 0.f;                      // lane s keeps choice s's weight (top <= 64)
+    int my_id = 0;
+    for (int s = 0; s < top; ++s) {
+        float best = -INFINITY;
+        int best_id = 0x7fffffff;
+        for (int e = lane; e < N; e += WAVE) {
+            const float v = cs[e];
+            if (v > best) { best = v; best_id = e; }
+        }
+#pragma unroll
+        for (int m = WAVE / 2; m > 0; m >>= 1) {
+            const float ov = __shfl_xor(best, m, WAVE);
+            const int oi = __shfl_xor(best_id, m, WAVE);
+            if (ov > best || (ov == best && oi < best_id)) { best = ov; best_id = oi; }
+        }
+        if (best_id >= N) best_id = s;                // NaN scores: still a valid output
+        const float w = expf(row[best_id] - zmax) / den;
+        sum += w;
+        if (lane == s) { mine = w; my_id = best_id; }
+        if (lane == best_id % WAVE) cs[best_id] = -INFINITY;
+    }
+    if (lane < top) {
+        ids[t * top + lane] = my_id;
+        wts[t * top + lane] = mine / (sum + 1e-20f);
+    }
+}
+
 __global__ void route_kernel(const float* __restrict__ z, int stride, int* __restrict__ ids, float* __restrict__ wts,
                              int n_tokens, int E, int top, int weight_fn) {
     const int t = blockIdx.x * blockDim.x + threadIdx.x;
@@ -177,6 +220,10 @@ __global__ __launch_bounds__(ROUTER_WAVES * WAVE) void router_kernel(const T* __
         }
     }
     __syncthreads();
+    if (weight_fn == 3) {
+        if (wave < nt) choose_corrected(zs + wave * N, cs + wave * E, ids, wts, t0 + wave, E, top, corr);
+        return;
+    }
     if (threadIdx.x < nt) {
         if (groups > 0) choose_limited(zs + threadIdx.x * N, cs + threadIdx.x * E, ids, wts, t0 + threadIdx.x, E, top, corr, groups, keep, scale);
         else choose(zs + threadIdx.x * N, ids, wts, t0 + threadIdx.x, E, top, weight_fn);
@@ -189,12 +236,13 @@ constexpr int ROWS_WG = 16;          // output rows a workgroup of four waves co
 // rounded to T as the second product takes it
 template <typename T>
 __global__ __launch_bounds__(256) void expert_up_kernel(const T* __restrict__ h, const T* __restrict__ w_up, const int* __restrict__ ids,
-                                                        const float* __restrict__ wts, T* __restrict__ a, int d, int F, int top,
+                                                        const float* __restrict__ wts, T* __restrict__ a, int d, int F, int top, int E,
                                                         int act, int scale_input, int gated, float limit, float alpha) {
     extern __shared__ float xs[];
     const long long row = blockIdx.x;
     const long long t = row / top;
     const int e = ids[row];
+    if (e >= E) return;                                   // an identity expert
     const float w = scale_input ? wts[row] : 1.f;
     for (int c = threadIdx.x; c < d; c += 256) xs[c] = to_f32(from_f32<T>(to_f32(h[t * d + c]) * w));
     __syncthreads();
@@ -219,10 +267,11 @@ __global__ __launch_bounds__(256) void expert_up_kernel(const T* __restrict__ h,
 // y[row][c] = W_down[e][c] . a[row]  (float32)
 template <typename T>
 __global__ __launch_bounds__(256) void expert_down_kernel(const T* __restrict__ a, const T* __restrict__ w_down, const int* __restrict__ ids,
-                                                          float* __restrict__ y, int d, int F) {
+                                                          float* __restrict__ y, int d, int F, int E) {
     extern __shared__ float as[];
     const long long row = blockIdx.x;
     const int e = ids[row];
+    if (e >= E) return;
     for (int f = threadIdx.x; f < F; f += 256) as[f] = to_f32(a[row * F + f]);
     __syncthreads();
     const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
@@ -235,15 +284,21 @@ __global__ __launch_bounds__(256) void expert_down_kernel(const T* __restrict__ 
     }
 }
 
-// residual[t][c] += sum over the token's choices, in their order, of y[t * top + s][c] (times the weight)
+// residual[t][c] += sum over the token's choices, in their order, of y[t * top + s][c] (times the weight); an identity
+// expert's choice (ids >= E, only where E > 0) adds the weight times h[t][c]
+template <typename T>
 __global__ void combine_kernel(const float* __restrict__ y, const float* __restrict__ wts, float* __restrict__ residual,
-                               long long n, int d, int top, int scale_output) {
+                               long long n, int d, int top, int scale_output, const int* __restrict__ ids, const T* __restrict__ h, int E) {
     const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n) return;
     const long long t = i / d;
     const int c = (int)(i - t * d);
     float acc = 0.f;
     for (int s = 0; s < top; ++s) {
+        if (E > 0 && ids[t * top + s] >= E) {
+            acc += to_f32(h[i]) * wts[t * top + s];
+            continue;
+        }
         const float v = y[(t * top + s) * d + c];
         acc += scale_output ? v * wts[t * top + s] : v;
     }
@@ -257,12 +312,14 @@ constexpr int GROUP_MAX_E = 1024;
 // One workgroup sorts the rows (token, choice) by expert and cuts each expert's rows into tiles of TM:
 // sorted[pos] = row; tiles[i] = (expert, first pos, rows), expert -1 for tiles beyond the last.  The order of an
 // expert's rows among themselves is whatever the atomics give: no row's result depends on its place in a tile.
+// (a choice e >= E, an identity expert's, is nobody's row)
 __global__ __launch_bounds__(1024) void group_rows_kernel(const int* __restrict__ ids, int R, int E, int TM, int* __restrict__ sorted,
                                                           int* __restrict__ tiles, int max_tiles) {
     __shared__ int cnt[GROUP_MAX_E], off[GROUP_MAX_E], cur[GROUP_MAX_E];
     for (int e = threadIdx.x; e < E; e += 1024) { cnt[e] = 0; cur[e] = 0; }
     __syncthreads();
-    for (int r = threadIdx.x; r < R; r += 1024) atomicAdd(&cnt[ids[r]], 1);
+    for (int r = threadIdx.x; r < R; r += 1024)
+        if (ids[r] < E) atomicAdd(&cnt[ids[r]], 1);
     __syncthreads();
     if (threadIdx.x == 0) {
         int o = 0, nt = 0;
@@ -278,7 +335,7 @@ __global__ __launch_bounds__(1024) void group_rows_kernel(const int* __restrict_
     __syncthreads();
     for (int r = threadIdx.x; r < R; r += 1024) {
         const int e = ids[r];
-        sorted[off[e] + atomicAdd(&cur[e], 1)] = r;
+        if (e < E) sorted[off[e] + atomicAdd(&cur[e], 1)] = r;
     }
 }
 
@@ -375,44 +432,48 @@ __global__ __launch_bounds__(256) void grouped_kernel(const bf16_t* __restrict__
 TUFF_EXPORT int tuff_moe_route(const float* z, int stride, int* ids, float* wts, int n_tokens, int E, int top, int weight_fn,
                                hipStream_t stream) {
     if (n_tokens <= 0) return 0;
-    if (top < 1 || top > E || stride < E) return -2;
+    if (top < 1 || top > E || stride < E || weight_fn < 0 || weight_fn > 2) return -2;
     hipLaunchKernelGGL(route_kernel, dim3(ceil_div(n_tokens, 64)), dim3(64), 0, stream, z, stride, ids, wts, n_tokens, E, top, weight_fn);
     return launch_status();
 }
 
+// ids: a choice of E and above is an identity expert's.
 // h [T][d], w_up [E][F][d] (gated: [E][2 F][d], an expert's gate rows then its up rows), w_down [E][d][F] of type dt; ids, wts [T][top]; a [T*top][F] (type dt) and
 // y [T*top][d] (float32) are work arrays; residual float32 [T][d].
 TUFF_EXPORT int tuff_moe_experts(const void* h, const void* w_up, const void* w_down, int dt, const int* ids, const float* wts,
-                                 void* a, float* y, float* residual, int n_tokens, int d, int F, int top, int act,
+                                 void* a, float* y, float* residual, int n_tokens, int d, int F, int E, int top, int act,
                                  int scale_input, int gated, float limit, float alpha, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
-    if (d > 16384 || F > 16384) return -2;
+    if (d > 16384 || F > 16384 || E < 1) return -2;
     const long long rows = (long long)n_tokens * top;
     dim3 block(256);
     if (dt == DT_F32) {
         hipLaunchKernelGGL(expert_up_kernel<float>, dim3((unsigned)rows, ceil_div(F, ROWS_WG)), block, d * sizeof(float), stream,
-                           (const float*)h, (const float*)w_up, ids, wts, (float*)a, d, F, top, act, scale_input, gated, limit, alpha);
+                           (const float*)h, (const float*)w_up, ids, wts, (float*)a, d, F, top, E, act, scale_input, gated, limit, alpha);
         hipLaunchKernelGGL(expert_down_kernel<float>, dim3((unsigned)rows, ceil_div(d, ROWS_WG)), block, F * sizeof(float), stream,
-                           (const float*)a, (const float*)w_down, ids, y, d, F);
+                           (const float*)a, (const float*)w_down, ids, y, d, F, E);
     } else {
         hipLaunchKernelGGL(expert_up_kernel<bf16_t>, dim3((unsigned)rows, ceil_div(F, ROWS_WG)), block, d * sizeof(float), stream,
-                           (const bf16_t*)h, (const bf16_t*)w_up, ids, wts, (bf16_t*)a, d, F, top, act, scale_input, gated, limit, alpha);
+                           (const bf16_t*)h, (const bf16_t*)w_up, ids, wts, (bf16_t*)a, d, F, top, E, act, scale_input, gated, limit, alpha);
         hipLaunchKernelGGL(expert_down_kernel<bf16_t>, dim3((unsigned)rows, ceil_div(d, ROWS_WG)), block, F * sizeof(float), stream,
-                           (const bf16_t*)a, (const bf16_t*)w_down, ids, y, d, F);
+                           (const bf16_t*)a, (const bf16_t*)w_down, ids, y, d, F, E);
     }
     const long long n = (long long)n_tokens * d;
-    hipLaunchKernelGGL(combine_kernel, dim3((unsigned)ceil_div_ll(n, 256)), block, 0, stream, y, wts, residual, n, d, top, !scale_input);
+    if (dt == DT_F32) hipLaunchKernelGGL(combine_kernel<float>, dim3((unsigned)ceil_div_ll(n, 256)), block, 0, stream, y, wts, residual, n, d, top, !scale_input, ids, (const float*)h, E);
+    else hipLaunchKernelGGL(combine_kernel<bf16_t>, dim3((unsigned)ceil_div_ll(n, 256)), block, 0, stream, y, wts, residual, n, d, top, !scale_input, ids, (const bf16_t*)h, E);
     return launch_status();
 }
 
 // z float32 [T][N], the first E columns the experts' logits; ids, wts [T][top].  W float32 [N][d]; h [T][d] of type dt.
 // bias float32 [E] or null: added to the experts' logits before the choice.  groups > 0: the limited choice (weight_fn 0),
-// with corr float32 [E] or null, `keep` of `groups` groups and the weights times `scale`; groups 0: the plain choice.
+// with corr float32 [E] or null, `keep` of `groups` groups and the weights times `scale`; groups 0: the plain choice, or,
+// weight_fn 3, the corrected one (top at most 64; identity experts are outputs like the others here).
 TUFF_EXPORT int tuff_moe_router(const void* h, int dt, const float* W, float* z, int* ids, float* wts, int n_tokens, int d,
                                 int N, int E, int top, int weight_fn, const float* bias, const float* corr, int groups, int keep,
                                 float scale, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
-    const int extra = groups > 0 ? E : 0;
+    const int extra = groups > 0 || weight_fn == 3 ? E : 0;
+    if (weight_fn == 3 && (groups > 0 || top > WAVE)) return -2;
     if (top < 1 || top > E || N < E || (long long)(d + 4 + N + extra) * 4 > 65536) return -2;
     if (groups > 0 && (weight_fn != 0 || groups > 64 || E % groups || keep < 1 || keep > groups || top > keep * (E / groups))) return -2;
     // long steps: four tokens a workgroup where that fits the LDS (the rows of W are then read a quarter as often)
@@ -629,7 +690,7 @@ TUFF_EXPORT int tuff_moe_experts_grouped(const void* h, const void* w_up, const 
         hipLaunchKernelGGL(grouped_tiled_kernel<false>, dim3(max_tiles, ceil_div(d, GT_BN)), dim3(GT_NT), lds, stream,
                            A_, (const bf16_t*)w_down, tiles, sorted, wts, nullptr, y, F, d, top, act, 0, 0, 0.f, 0.f);
         const long long n = (long long)n_tokens * d;
-        hipLaunchKernelGGL(combine_kernel, dim3((unsigned)ceil_div_ll(n, 256)), dim3(256), 0, stream, y, wts, residual, n, d, top, !scale_input);
+        hipLaunchKernelGGL(combine_kernel<bf16_t>, dim3((unsigned)ceil_div_ll(n, 256)), dim3(256), 0, stream, y, wts, residual, n, d, top, !scale_input, ids, H_, E);
         return launch_status();
     }
     hipLaunchKernelGGL(group_rows_kernel, dim3(1), dim3(1024), 0, stream, ids, (int)R, E, TM, sorted, tiles, max_tiles);
@@ -651,6 +712,6 @@ TUFF_EXPORT int tuff_moe_experts_grouped(const void* h, const void* w_up, const 
                            A_, (const bf16_t*)w_down, tiles, sorted, wts, nullptr, y, F, d, top, act, scale_input, 0, 0.f, 0.f);
     }
     const long long n = (long long)n_tokens * d;
-    hipLaunchKernelGGL(combine_kernel, dim3((unsigned)ceil_div_ll(n, 256)), dim3(256), 0, stream, y, wts, residual, n, d, top, !scale_input);
+    hipLaunchKernelGGL(combine_kernel<bf16_t>, dim3((unsigned)ceil_div_ll(n, 256)), dim3(256), 0, stream, y, wts, residual, n, d, top, !scale_input, ids, H_, E);
     return launch_status();
 }

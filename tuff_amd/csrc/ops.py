@@ -27,7 +27,7 @@ class KernelError(RuntimeError):
 
 _SIGNATURES = {
     "elementwise": {
-        "tuff_embed_rows": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_float, _c_void_p],
+        "tuff_embed_rows": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_float, _c_void_p],
         "tuff_add_bias": [_c_void_p, _c_int, _c_void_p, _c_ll, _c_int, _c_void_p],
         "tuff_scale_cap": [_c_void_p, _c_ll, _c_float, _c_float, _c_void_p],
         "tuff_rmsnorm": [_c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_ll, _c_float, _c_void_p],
@@ -40,6 +40,7 @@ _SIGNATURES = {
         "tuff_dyt": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_void_p],
         "tuff_glu": [_c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_float, _c_float, _c_void_p],
         "tuff_act_rows": [_c_void_p, _c_int, _c_void_p, _c_int, _c_ll, _c_int, _c_int, _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p],
+        "tuff_act_lookup": [_c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_ll, _c_int, _c_int, _c_int, _c_ll, _c_int, _c_void_p],
         "tuff_pad_cols": [_c_void_p, _c_void_p, _c_int, _c_ll, _c_int, _c_int, _c_void_p],
     },
     "recurrent": {
@@ -74,7 +75,7 @@ _SIGNATURES = {
         "tuff_moe_experts_grouped": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p,
                                      _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_void_p],
         "tuff_moe_experts": [_c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
-                             _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_void_p],
+                             _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_void_p],
     },
     "gemm_f32": {
         "tuff_gemm_f32": [_c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p],
@@ -101,13 +102,16 @@ _SIGNATURES = {
                           _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p,
                           _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_int, _c_int, _c_void_p],
         "tuff_rope_table": [_c_void_p, _c_int, _c_int, _c_void_p, _c_void_p],
+        "tuff_qkv_rotate_write": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int,
+                                  _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_int, _c_void_p],
         "tuff_kv_write": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p,
                           _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
     },
     "attention": {
         "tuff_attention_general": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int,
                                    _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                                   _c_float, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_void_p],
+                                   _c_float, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+        "tuff_diff_combine": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void_p],
         "tuff_attention_decode_exact": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p,
                                         _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
                                         _c_int, _c_float, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
@@ -116,14 +120,14 @@ _SIGNATURES = {
                                _c_void_p],
     },
     "attention_single": {
-        "tuff_attention_single_plan": [_c_int, _c_int, _c_int, _c_int, _c_int, ctypes.POINTER(_c_int), ctypes.POINTER(_c_int)],
+        "tuff_attention_single_plan": [_c_int, _c_int, _c_int, _c_int, _c_int, _c_int, ctypes.POINTER(_c_int), ctypes.POINTER(_c_int)],
         "tuff_attention_single": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p,
                                   _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void_p, _c_void_p,
-                                  _c_int, _c_int, _c_void_p],
+                                  _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void_p],
     },
     "postnorm": {
         "tuff_post_norm_add": [_c_void_p, _c_void_p, _c_void_p, _c_float, _c_float, _c_void_p, _c_void_p, _c_float, _c_void_p,
-                               _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p],
+                               _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p],
         "tuff_normed_mean2": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_float, _c_float, _c_void_p, _c_int, _c_int, _c_void_p],
         "tuff_scale_add_layer_norm": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_float, _c_void_p, _c_int, _c_void_p, _c_int, _c_int,
                                       _c_int, _c_void_p],
@@ -180,7 +184,10 @@ _SIGNATURES = {
                                           _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p],
         "tuff_attention_prefill_wide": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int,
                                         _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
-                                        _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p],
+                                        _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p],
+        "tuff_attention_prefill_diff": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_void_p,
+                                        _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_float, _c_void_p],
+        "tuff_attention_prefill_diff_block_columns": [],
         "tuff_attention_prefill_block_columns": [_c_int],
     },
     "shortconv": {
@@ -342,11 +349,11 @@ def _check(code: int, what: str) -> None:
 
 # ------------------------------------------------------------------------ row kernels
 def embed_rows(table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor, scale: float = 1.0) -> None:
-    """out[t] = table[tokens[t]] * scale, float32."""
+    """out[t] = table[tokens[t]] * scale, in out's type (float32 for the residual stream)."""
     n, d = out.shape
     _check(load("elementwise").tuff_embed_rows(
         _gpu("table", table, shape=(None, d)), _dt(table), _gpu("tokens", tokens, torch.int32, (n,)),
-        _gpu("out", out, torch.float32), n, d, float(scale), _stream()), "embed_rows")
+        _gpu("out", out), _dt(out), n, d, float(scale), _stream()), "embed_rows")
 
 
 def add_bias(y: torch.Tensor, bias: torch.Tensor) -> None:
@@ -480,6 +487,20 @@ def act_rows(inp: torch.Tensor, out: torch.Tensor, activation: str, row_gate: Op
         inp.data_ptr(), _dt(inp), out.data_ptr(), _dt(out), rows, N, kind, gp, stride,
         -1 if gate_activation is None else ACTIVATIONS[gate_activation], _opt("bias", bias, torch.float32, (N,)),
         _opt("params", params, torch.float32, (2,)), _stream()), "act_rows")
+
+
+def act_lookup(inp: torch.Tensor, table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor, activation: str, col0: int = 0) -> None:
+    """out[t, c] = activation(inp[t, c]) * table[tokens[t], col0 + c], inp float32 [T, N]; out [T, >= N], zeros beyond N.  tokens
+    int32 [T], ids within the table."""
+    T, N = inp.shape
+    _gpu("inp", inp, torch.float32)
+    _gpu("out", out, shape=(T, None))
+    _gpu("table", table)
+    if table.dim() != 2 or col0 < 0 or col0 + N > table.shape[1] or out.shape[1] < N:
+        raise KernelError(f"act_lookup: {N} columns from {col0} of a table of {tuple(table.shape)} into {tuple(out.shape)}")
+    _check(load("elementwise").tuff_act_lookup(
+        inp.data_ptr(), table.data_ptr(), _dt(table), _gpu("tokens", tokens, torch.int32, (T,)), out.data_ptr(), _dt(out), T, N,
+        out.shape[1], ACTIVATIONS[activation], table.shape[1], int(col0), _stream()), "act_lookup")
 
 
 def pad_cols(inp: torch.Tensor, width: int) -> torch.Tensor:
@@ -842,6 +863,40 @@ def qkv_post(qkv, q_out, *, H, Hkv, hd, positions, eps=0.0, q_norm_w=None, k_nor
         qkv.shape[1] if wide_rows else 0, _stream()), "qkv_post")
 
 
+def qkv_rotate_write(qkv, q_out, *, H, Hk, hd, vd, positions, maps: int = 1, bias=None, inv_freq=None, rotary_dim: int = 0,
+                     k_cache=None, v_cache=None, slot_mapping=None, page_size: int = 1, angles=None) -> None:
+    """qkv float32 [T, (H + Hk) hd + (Hk / maps) vd], the sums of a projection: adds the bias (float32, a row's width, or None),
+    rotates q and k (halves of the first rotary_dim channels pair up) and writes the caches.  A cached key row holds `maps`
+    keys of hd channels side by side: k_cache [P, Hk / maps, page, maps hd], v_cache [P, Hk / maps, vd, page].  q_out [T, H hd]
+    of the caches' type."""
+    T = qkv.shape[0]
+    if Hk % maps:
+        raise KernelError(f"qkv_rotate_write: {Hk} key heads in rows of {maps}")
+    G = Hk // maps
+    width = (H + Hk) * hd + G * vd
+    _gpu("qkv", qkv, torch.float32, (T, width))
+    _opt("bias", bias, torch.float32, (width,))
+    _gpu("q_out", q_out, shape=(T, H * hd))
+    if (k_cache is None) != (v_cache is None) or (k_cache is not None and slot_mapping is None):
+        raise KernelError("qkv_rotate_write: both caches and a slot mapping, or none of them")
+    if k_cache is not None:
+        P = k_cache.shape[0]
+        _gpu("k_cache", k_cache, q_out.dtype, (P, G, page_size, maps * hd))
+        _gpu("v_cache", v_cache, q_out.dtype, (P, G, vd, page_size))
+        _gpu("slot_mapping", slot_mapping, torch.int32, (T,))
+    if rotary_dim:
+        if rotary_dim < 0 or rotary_dim > hd or rotary_dim % 2:
+            raise KernelError(f"qkv_rotate_write: rotary_dim {rotary_dim} must be even and within the head size {hd}")
+        _gpu("inv_freq", inv_freq, torch.float32, (rotary_dim // 2,))
+        _opt("angles", angles, torch.float32, (None, 2, rotary_dim // 2))
+    _gpu("positions", positions, torch.int32, (T,))
+    p = lambda t: None if t is None else t.data_ptr()
+    _check(load("rope_kv").tuff_qkv_rotate_write(
+        qkv.data_ptr(), p(bias), q_out.data_ptr(), p(k_cache), p(v_cache), _dt(q_out), p(inv_freq) if rotary_dim else None, int(rotary_dim),
+        positions.data_ptr(), p(slot_mapping), T, H, Hk, hd, maps, vd, page_size, p(angles) if rotary_dim else None,
+        0 if angles is None or not rotary_dim else angles.shape[0], _stream()), "qkv_rotate_write")
+
+
 def rope_table(inv_freq: torch.Tensor, n_pos: int) -> torch.Tensor:
     """float32 [n_pos, 2, len(inv_freq)]: cosines and sines of pos * inv_freq, bit for bit what the
     rotation kernels compute for themselves."""
@@ -871,18 +926,24 @@ def kv_write(k, v, k_cache, v_cache, slot_mapping, *, Hkv, hd, page_size, vd=Non
 # -------------------------------------------------------------------------- attention
 def attention_general(q, k_cache, v_cache, out, *, block_table, req_of_token, positions,
                       H, Hkv, hd, page_size, window=0, scale=None, vd=None, sinks=None, slopes=None,
-                      log_distance=None, all_values: bool = False) -> None:
+                      log_distance=None, all_values: bool = False, keep_first: int = 0, maps: int = 1) -> None:
     """vd: width of a value where it is not the keys'.  sinks: float32 [H], a logit per head that counts
     once in the softmax's denominator and has no value.  slopes: float32 [H]; slopes[h] * (position - key) is
     taken off head h's scaled scores.  v_cache None: the values are the first vd channels of the key rows.
     log_distance: (r1, r2), float32 [H] each; r1[h] * ln(1 + r2[h] * (position - key)) is taken off head h's scaled
     scores.  all_values: every query head's weights are applied to the values of every kv head; out is then float32
-    [T, H * Hkv * vd] (head, kv head, channel), for head_mix_gate."""
+    [T, H * Hkv * vd] (head, kv head, channel), for head_mix_gate.  keep_first: with a window, keys before it are seen
+    whatever the distance.  maps: a key row of hd channels holds that many keys side by side; H counts maps, head h's query
+    (hd / maps channels) meets part h % maps, and out may be float32 whatever q's type (for diff_combine)."""
     T = q.shape[0]
     dt = q.dtype
     vd = hd if vd is None else int(vd)
-    _gpu("q", q, shape=(T, H * hd))
-    if all_values:
+    if maps < 1 or hd % maps or H % maps:
+        raise KernelError(f"attention: {maps} maps of {H} heads in key rows of {hd} channels")
+    _gpu("q", q, shape=(T, H * (hd // maps)))
+    if maps > 1:
+        _gpu("out", out, out.dtype if out.dtype == torch.float32 else dt, (T, H * vd))
+    elif all_values:
         if v_cache is None:
             raise KernelError("attention: all_values needs a value cache")
         _gpu("out", out, torch.float32, (T, H * Hkv * vd))
@@ -916,7 +977,18 @@ def attention_general(q, k_cache, v_cache, out, *, block_table, req_of_token, po
         block_table.data_ptr(), block_table.shape[1], req_of_token.data_ptr(), positions.data_ptr(),
         T, H, Hkv, hd, vd, page_size, int(window or 0), float(scale), None if sinks is None else sinks.data_ptr(),
         None if slopes is None else slopes.data_ptr(), int(v_cache is None),
-        None if r1 is None else r1.data_ptr(), None if r2 is None else r2.data_ptr(), int(all_values), _stream()), "attention_general")
+        None if r1 is None else r1.data_ptr(), None if r2 is None else r2.data_ptr(), int(all_values),
+        int(keep_first) if window else 0, int(maps), int(maps > 1 and out.dtype == torch.float32), _stream()), "attention_general")
+
+
+def diff_combine(o, out, *, H, vd, combine) -> None:
+    """A head's two maps (o float32 [T, 2 H vd], side by side) into its output: combine = (lambda, eps, coef),
+    v = a1 - lambda a2, out [T, H vd] = v / sqrt(mean(v^2) + eps) * coef over the head's channels."""
+    T = o.shape[0]
+    lam, eps, coef = combine
+    _check(load("attention").tuff_diff_combine(
+        _gpu("o", o, torch.float32, (T, 2 * H * vd)), _gpu("out", out, shape=(T, H * vd)), _dt(out), T, H, vd,
+        float(lam), float(eps), float(coef), _stream()), "diff_combine")
 
 
 def head_mix_gate(o, out, *, H, Hkv, vd, talk=None, gates=None) -> None:
@@ -944,29 +1016,35 @@ def head_mix_gate(o, out, *, H, Hkv, vd, talk=None, gates=None) -> None:
 
 # ------------------------------------------------- sublayers normed before they join the stream
 def post_norm_add(x, *, y=None, w=None, eps: float = 0.0, mult: float = 1.0, extra=None, next_w=None, next_eps: float = 0.0,
-                  h_out=None, clear_y: bool = False, y_next=None) -> None:
+                  h_out=None, clear_y: bool = False, y_next=None, y_bias=None, row=None) -> None:
     """One kernel over the residual stream x (float32 [T, d], in place).  With y float32 [T, d] and w float32 [d]:
     x <- x + mult * y / sqrt(mean(y^2) + eps) * w (y is then cleared, if asked).  With extra float32 [T, d]:
     x <- x + extra.  With next_w float32 [d] and h_out [T, d]: h_out = x / sqrt(mean(x^2) + next_eps) * next_w,
     from the new x.  y_next float32 [d] (with clear_y): every row of y is left holding y_next instead of zeros, the bias of
-    the product that adds into y next."""
+    the product that adds into y next.  y_bias float32 [d]: y lacks a bias, which is added first.  row float32 [d]: added to
+    every row of x.  h_out without next_w: the new x itself, rounded to h_out's type."""
     T, d = x.shape
+    _opt("y_bias", y_bias, torch.float32, (d,))
+    _opt("row", row, torch.float32, (d,))
+    if y_bias is not None and y is None:
+        raise KernelError("post_norm_add: a bias of y without y")
     _opt("y_next", y_next, torch.float32, (d,))
     _gpu("x", x, torch.float32, (T, d))
     _opt("y", y, torch.float32, (T, d))
     if y is not None:
         _gpu("w", w, torch.float32, (d,))
     _opt("extra", extra, torch.float32, (T, d))
-    if (next_w is None) != (h_out is None):
-        raise KernelError("post_norm_add: next_w and h_out go together")
-    if next_w is not None:
-        _gpu("next_w", next_w, torch.float32, (d,))
+    if next_w is not None and h_out is None:
+        raise KernelError("post_norm_add: next_w without h_out")
+    if h_out is not None:
+        _opt("next_w", next_w, torch.float32, (d,))
         _gpu("h_out", h_out, shape=(T, d))
     _check(load("postnorm").tuff_post_norm_add(
         x.data_ptr(), None if y is None else y.data_ptr(), None if y is None else w.data_ptr(), float(eps), float(mult),
         None if extra is None else extra.data_ptr(), None if next_w is None else next_w.data_ptr(), float(next_eps),
         None if h_out is None else h_out.data_ptr(), DT_F32 if h_out is None else _dt(h_out), T, d, int(clear_y),
-        None if y_next is None else y_next.data_ptr(), _stream()),
+        None if y_next is None else y_next.data_ptr(), None if y_bias is None else y_bias.data_ptr(),
+        None if row is None else row.data_ptr(), _stream()),
         "post_norm_add")
 
 
@@ -1477,30 +1555,37 @@ def attention_single_supported(dtype, hd: int, vd: int, page_size: int) -> bool:
 _single_plans: dict = {}
 
 
-def attention_single_plan(T: int, H: int, Hkv: int, max_ctx_len: int, window: int) -> tuple:
+def attention_single_plan(T: int, H: int, Hkv: int, max_ctx_len: int, window: int, keep_first: int = 0) -> tuple:
     """(keys a part, parts a token) of attention_single for T tokens."""
-    key = (T, H, Hkv, max_ctx_len, window)
+    key = (T, H, Hkv, max_ctx_len, window, keep_first)
     if key not in _single_plans:
         if len(_single_plans) > 4096:
             _single_plans.clear()
         pk, n = _c_int(0), _c_int(0)
-        _check(load("attention_single").tuff_attention_single_plan(T, H, Hkv, max_ctx_len, window, ctypes.byref(pk), ctypes.byref(n)),
+        _check(load("attention_single").tuff_attention_single_plan(T, H, Hkv, max_ctx_len, window, keep_first, ctypes.byref(pk), ctypes.byref(n)),
                "attention_single_plan")
         _single_plans[key] = (int(pk.value), int(n.value))
     return _single_plans[key]
 
 
 def attention_single(q, k_cache, v_cache, out, *, block_table, req_of_token, positions, H, Hkv, hd, vd, page_size, max_ctx_len,
-                     window=0, scale=None, sinks=None, slopes=None) -> None:
+                     window=0, scale=None, sinks=None, slopes=None, keep_first: int = 0, combine=None) -> None:
     """Single tokens over the bfloat16 cache on the matrix cores with float32-precise softmax weights (each goes through
     the products as two bfloat16 numbers).  out [T, H * vd], bfloat16 or float32.  sinks, slopes: float32 [H] or None, as for
-    attention_general."""
+    attention_general.  keep_first: with a window, keys before it are seen whatever the distance.  combine = (lambda, eps,
+    coef): differential attention; a key row of hd channels holds two keys, H counts maps (a head's two side by side), q is
+    [T, H * hd / 2] and out [T, H / 2 * vd] what diff_combine makes of a head's maps."""
     T = q.shape[0]
+    maps = 1 if combine is None else 2
+    keep_first = int(keep_first) if window else 0
     if not attention_single_supported(q.dtype, hd, vd, page_size):
         raise KernelError(f"attention_single: bfloat16, head sizes that are multiples of 8 up to 256 (got {hd}, {vd}) and a page size "
                           f"that is a multiple of 16 (got {page_size})")
-    _gpu("q", q, torch.bfloat16, (T, H * hd))
-    _gpu("out", out, shape=(T, H * vd))
+    if maps == 2 and (hd % 16 or H % Hkv or (H // Hkv) % 2 or sinks is not None):
+        raise KernelError(f"attention_single: two maps a head need keys of a multiple of 8 channels (rows of {hd}), an even number of "
+                          f"maps a kv head ({H}:{Hkv}) and no sinks")
+    _gpu("q", q, torch.bfloat16, (T, H * (hd // maps)))
+    _gpu("out", out, shape=(T, H // maps * vd))
     P = k_cache.shape[0]
     _gpu("k_cache", k_cache, torch.bfloat16, (P, Hkv, page_size, hd))
     _gpu("v_cache", v_cache, torch.bfloat16, (P, Hkv, vd, page_size))
@@ -1515,14 +1600,15 @@ def attention_single(q, k_cache, v_cache, out, *, block_table, req_of_token, pos
         raise KernelError("attention_single: the query heads must be a multiple of the kv heads")
     if scale is None:
         scale = 1.0 / math.sqrt(hd)
-    part_keys, n_slots = attention_single_plan(T, H, Hkv, int(max_ctx_len), int(window or 0))
+    part_keys, n_slots = attention_single_plan(T, H, Hkv, int(max_ctx_len), int(window or 0), keep_first)
     ws_o = torch.empty(T * H * n_slots * vd, dtype=torch.float32, device=q.device)
     ws_ml = torch.empty(T * H * n_slots * 2, dtype=torch.float32, device=q.device)
     ptr = lambda x: None if x is None else x.data_ptr()
     _check(load("attention_single").tuff_attention_single(
         q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(), _dt(out), ws_o.data_ptr(), ws_ml.data_ptr(),
         block_table.data_ptr(), block_table.shape[1], req_of_token.data_ptr(), positions.data_ptr(), T, H, Hkv, hd, vd, page_size,
-        int(window or 0), float(scale), ptr(sinks), ptr(slopes), part_keys, n_slots, _stream()), "attention_single")
+        int(window or 0), float(scale), ptr(sinks), ptr(slopes), part_keys, n_slots, keep_first, maps,
+        *(float(v) for v in (combine or (0.0, 0.0, 0.0))), _stream()), "attention_single")
 
 
 def attention_prefill_wide_supported(dtype, hd: int, vd: int, page_size: int) -> bool:
@@ -1530,12 +1616,14 @@ def attention_prefill_wide_supported(dtype, hd: int, vd: int, page_size: int) ->
 
 
 def attention_prefill_wide(q, k_cache, v_cache, out, *, block_table, blocks, req_info, H, Hkv, hd, vd, page_size, max_ctx_len,
-                           window=0, scale=None, sinks=None, slopes=None, log_distance=None, all_values: bool = False) -> None:
+                           window=0, scale=None, sinks=None, slopes=None, log_distance=None, all_values: bool = False,
+                           keep_first: int = 0) -> None:
     """attention_prefill's kernel in its wide form: values of vd channels (v_cache [P, Hkv, vd, page_size]), softmax
     weights that keep float32's precision through the matrix cores, and optionally log_distance = (r1, r2), float32 [H]
     each: r1[h] * ln(1 + r2[h] * (position - key)) is taken off head h's scaled scores.  all_values: every query head's
     weights are applied to the values of every kv head and out is float32 [T, H * Hkv * vd] (head, kv head, channel), for
-    head_mix_gate; otherwise out is bfloat16 [T, H * vd].  The keys are not cut into segments."""
+    head_mix_gate; otherwise out is bfloat16 [T, H * vd].  The keys are not cut into segments.  keep_first: with a window, keys
+    before it are seen whatever the distance."""
     T = q.shape[0]
     if not attention_prefill_wide_supported(q.dtype, hd, vd, page_size):
         raise KernelError(f"attention_prefill_wide: needs bfloat16, head sizes that are multiples of 8 (got {hd}, {vd}) "
@@ -1577,8 +1665,47 @@ def attention_prefill_wide(q, k_cache, v_cache, out, *, block_table, blocks, req
         q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(), block_table.data_ptr(), block_table.shape[1],
         None if blocks is None else blocks.data_ptr(), nblk, req_info.data_ptr(), H, Hkv, hd, vd, page_size, int(window or 0),
         float(scale), None if sinks is None else sinks.data_ptr(), None if slopes is None else slopes.data_ptr(),
-        None if r1 is None else r1.data_ptr(), None if r2 is None else r2.data_ptr(), int(bool(all_values)), _stream()),
-        "attention_prefill_wide")
+        None if r1 is None else r1.data_ptr(), None if r2 is None else r2.data_ptr(), int(bool(all_values)),
+        int(keep_first) if window else 0, _stream()), "attention_prefill_wide")
+
+
+def attention_prefill_diff_supported(dtype, dim: int, vd: int, page_size: int) -> bool:
+    return dtype == torch.bfloat16 and dim % 8 == 0 and vd % 8 == 0 and dim <= 128 and vd <= 256 and page_size % 16 == 0
+
+
+def attention_prefill_diff_block_columns() -> int:
+    return int(load("attention_prefill").tuff_attention_prefill_diff_block_columns())
+
+
+def attention_prefill_diff(q, k_cache, v_cache, out, *, block_table, blocks, req_info, heads, Hkv, dim, vd, page_size, max_ctx_len,
+                           combine, window=0, keep_first: int = 0, scale) -> None:
+    """Differential attention of steps with prompt portions: q [T, heads * 2 * dim] (a head's two maps side by side), k_cache
+    [P, Hkv, page, 2 dim], v_cache [P, Hkv, vd, page], out bfloat16 [T, heads * vd] = what diff_combine makes of a head's maps
+    with combine = (lambda, eps, coef).  Softmax weights keep float32's precision.  blocks: query_blocks() of heads / Hkv
+    columns a token in blocks of attention_prefill_diff_block_columns()."""
+    T = q.shape[0]
+    if not attention_prefill_diff_supported(q.dtype, dim, vd, page_size):
+        raise KernelError(f"attention_prefill_diff: bfloat16, keys of a multiple of 8 channels up to 128 (got {dim}), values of one up to 256 "
+                          f"(got {vd}) and a page size that is a multiple of 16 (got {page_size})")
+    _gpu("q", q, torch.bfloat16, (T, heads * 2 * dim))
+    _gpu("out", out, torch.bfloat16, (T, heads * vd))
+    P = k_cache.shape[0]
+    _gpu("k_cache", k_cache, torch.bfloat16, (P, Hkv, page_size, 2 * dim))
+    _gpu("v_cache", v_cache, torch.bfloat16, (P, Hkv, vd, page_size))
+    _gpu("block_table", block_table, torch.int32)
+    R = req_info.shape[0]
+    _gpu("req_info", req_info, torch.int32, (R, 4))
+    if block_table.dim() != 2 or block_table.shape[0] != R or block_table.shape[1] * page_size < int(max_ctx_len):
+        raise KernelError("attention_prefill_diff: block_table must be [requests, blocks] and cover the longest context")
+    if heads % Hkv:
+        raise KernelError("attention_prefill_diff: the heads must be a multiple of the kv heads")
+    nblk = blocks.shape[0]
+    _gpu("blocks", blocks, torch.int32, (nblk, 2))
+    lam, eps, coef = combine
+    _check(load("attention_prefill").tuff_attention_prefill_diff(
+        q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(), block_table.data_ptr(), block_table.shape[1],
+        blocks.data_ptr(), nblk, req_info.data_ptr(), heads, Hkv, dim, vd, page_size, int(window or 0), int(keep_first) if window else 0,
+        float(scale), float(lam), float(eps), float(coef), _stream()), "attention_prefill_diff")
 
 
 def query_blocks(q_len, G: int, nb: int, ctx_len=None):
@@ -1882,7 +2009,7 @@ def head_norm_gate(o, w, gate, out, *, H, Dv, eps, per_head_weight: bool, gate_a
 
 
 # ------------------------------------------------------------------ mixture of experts
-ROUTER_WEIGHTS = {"sigmoid": 0, "softmax": 1, "softmax_all": 2}
+ROUTER_WEIGHTS = {"sigmoid": 0, "softmax": 1, "softmax_all": 2, "softmax_share": 3}       # (softmax_share: moe_router only)
 
 
 def moe_route(z, ids, wts, *, E, top, weights: str = "sigmoid") -> None:
@@ -1907,10 +2034,18 @@ def moe_router(h, w, z, ids, wts, *, E, top, weights: str = "sigmoid", bias=None
     E columns, the choice as moe_route makes it, in one kernel.  bias: float32 [E], added to the experts' logits.
     groups > 0 (sigmoid weights): a limited choice.  It runs on sigmoid(z) + correction (float32 [E] or None) and only
     inside the `keep` groups, of `groups` equal groups of neighbouring experts, whose two largest such scores have the
-    largest sum; the weights are sigmoid(z) of the chosen, without the correction, times `scale`."""
+    largest sum; the weights are sigmoid(z) of the chosen, without the correction, times `scale`.
+    weights "softmax_share": the choice runs on softmax(z over all E) + correction, and the weights are the chosen ones'
+    softmax, without the correction, divided by their sum.  (E counts every output a choice may fall on, identity experts
+    included.)"""
     T, d = h.shape
     N = w.shape[0]
-    if d + N + (E if groups else 0) > ROUTER_MAX_FLOATS:
+    share = weights == "softmax_share"
+    if share and (groups or top > 64):
+        raise KernelError(f"moe_router: shares of the softmax go with no groups and at most 64 choices, got {groups} and {top}")
+    if correction is not None and not groups and not share:
+        raise KernelError("moe_router: a correction goes with a limited choice or with shares of the softmax")
+    if d + N + (E if groups or share else 0) > ROUTER_MAX_FLOATS:
         raise KernelError(f"moe_router: hidden size {d} + {N} logits above {ROUTER_MAX_FLOATS}")
     if groups and (weights != "sigmoid" or groups > 64 or E % groups or not 1 <= keep <= groups or top > keep * (E // groups)):
         raise KernelError(f"moe_router: a limited choice of {top} among {keep} of {groups} groups of {E} experts is not possible")
@@ -1949,7 +2084,8 @@ def moe_experts_grouped(h, up_tiles, down_tiles, ids, wts, residual, *, F: int, 
                         scale_input: bool = True, gated: bool = False, limit: float = 0.0, alpha: float = 1.0) -> None:
     """moe_experts on the matrix cores, bfloat16: the rows (token, choice) are sorted by expert and every expert's
     rows go through its two matrices in tiles.  up_tiles, down_tiles: tile_experts() of the [F, d] and [d, F] matrices;
-    gated: of interleave_gate_up(gate, up) [2 F, d] and [d, F]."""
+    gated: of interleave_gate_up(gate, up) [2 F, d] and [d, F].  A choice in ids beyond the last expert is an identity expert's:
+    it adds the weight times h[t]."""
     T, d = h.shape
     E, top = up_tiles.shape[0], ids.shape[1]
     if not moe_grouped_supported(h.dtype, d, F, E):
@@ -1980,7 +2116,8 @@ def moe_experts(h, w_up, w_down, ids, wts, residual, *, activation: str = "relu2
                 gated: bool = False, limit: float = 0.0, alpha: float = 1.0) -> None:
     """residual[t] += sum over the token's choices of W_down[e] act(W_up[e] x), x = h[t] times the choice's
     weight (scale_input) or the product times it.  h [T, d]; w_up [E, F, d]; w_down [E, d, F], all of one type.
-    gated: w_up is [E, 2 F, d], an expert's gate rows then its up rows, and the activation joins the two."""
+    gated: w_up is [E, 2 F, d], an expert's gate rows then its up rows, and the activation joins the two.  A choice in ids
+    beyond the last expert is an identity expert's: it adds the weight times h[t]."""
     T, d = h.shape
     E, F, _ = w_up.shape
     if gated:
@@ -1998,7 +2135,7 @@ def moe_experts(h, w_up, w_down, ids, wts, residual, *, activation: str = "relu2
     a = torch.empty(T * top, F, dtype=dt, device=h.device)
     y = torch.empty(T * top, d, dtype=torch.float32, device=h.device)
     _check(load("moe").tuff_moe_experts(h.data_ptr(), w_up.data_ptr(), w_down.data_ptr(), _dt(h), ids.data_ptr(),
-                                        wts.data_ptr(), a.data_ptr(), y.data_ptr(), residual.data_ptr(), T, d, F, top,
+                                        wts.data_ptr(), a.data_ptr(), y.data_ptr(), residual.data_ptr(), T, d, F, E, top,
                                         _expert_activation(activation, gated, limit), int(scale_input), int(gated),
                                         float(limit), float(alpha), _stream()),
            "moe_experts")

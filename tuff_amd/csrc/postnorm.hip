@@ -1,9 +1,11 @@
 // Kernels of layers that norm a sublayer's output before it joins the residual stream, all in float32.
 //
 // tuff_post_norm_add, a workgroup a token:
-//     x <- x + mult * y / sqrt(mean(y^2) + eps) * w  [+ extra]        (y is then cleared, if asked, or set to a row
+//     x <- x + mult * y / sqrt(mean(y^2) + eps) * w  [+ extra] [+ row]   (y is then cleared, if asked, or set to a row
 //                                                                      y_next: the bias of the product that adds into y next)
-//     h  = x / sqrt(mean(x^2) + eps_next) * w_next                     (if asked: the next sublayer's input)
+//     h  = x / sqrt(mean(x^2) + eps_next) * w_next                     (if asked: the next sublayer's input; without a
+//                                                                      weight h is x itself, rounded to its type)
+// y may lack a bias, a row y_bias that is added to it before anything else.
 // One launch where a norm, a residual sum, another sum and the next norm would be four.  Without y only the
 // sum with `extra` and the next norm run.  The weights come in as float32 with any offset already added.
 //
@@ -30,7 +32,7 @@ template <typename T>
 __global__ __launch_bounds__(PN_THREADS) void post_norm_add_kernel(
     float* __restrict__ x, float* __restrict__ y, const float* __restrict__ w, float eps, float mult,
     const float* __restrict__ extra, const float* __restrict__ w_next, float eps_next, T* __restrict__ h_out,
-    int d, int clear_y, const float* __restrict__ y_next) {
+    int d, int clear_y, const float* __restrict__ y_next, const float* __restrict__ y_bias, const float* __restrict__ row_add) {
     __shared__ float scratch[PN_WAVES];
     const long long row = (long long)blockIdx.x * d;
     float* xr = x + row;
@@ -38,7 +40,10 @@ __global__ __launch_bounds__(PN_THREADS) void post_norm_add_kernel(
     if (y) {
         const float* yr = y + row;
         float ss = 0.f;
-        for (int c = threadIdx.x; c < d; c += PN_THREADS) ss = fmaf(yr[c], yr[c], ss);
+        for (int c = threadIdx.x; c < d; c += PN_THREADS) {
+            const float v = y_bias ? yr[c] + y_bias[c] : yr[c];
+            ss = fmaf(v, v, ss);
+        }
         ss = block_sum<PN_WAVES>(ss, scratch);
         inv = mult / sqrtf(ss / (float)d + eps);
     }
@@ -46,14 +51,19 @@ __global__ __launch_bounds__(PN_THREADS) void post_norm_add_kernel(
     for (int c = threadIdx.x; c < d; c += PN_THREADS) {
         float v = xr[c];
         if (y) {
-            v = fmaf(y[row + c] * inv, w[c], v);
+            v = fmaf((y_bias ? y[row + c] + y_bias[c] : y[row + c]) * inv, w[c], v);
             if (clear_y) y[row + c] = y_next ? y_next[c] : 0.f;
         }
         if (extra) v += extra[row + c];
-        if (y || extra) xr[c] = v;
+        if (row_add) v += row_add[c];
+        if (y || extra || row_add) xr[c] = v;
         ss2 = fmaf(v, v, ss2);
     }
     if (!h_out) return;
+    if (!w_next) {
+        for (int c = threadIdx.x; c < d; c += PN_THREADS) h_out[row + c] = from_f32<T>(xr[c]);
+        return;
+    }
     ss2 = block_sum<PN_WAVES>(ss2, scratch);
     const float inv2 = 1.0f / sqrtf(ss2 / (float)d + eps_next);
     // (a thread reads back the elements it wrote itself)
@@ -67,19 +77,21 @@ template <typename T, int EPT>
 __global__ __launch_bounds__(PN_THREADS) void post_norm_add_regs_kernel(
     float* __restrict__ x, float* __restrict__ y, const float* __restrict__ w, float eps, float mult,
     const float* __restrict__ extra, const float* __restrict__ w_next, float eps_next, T* __restrict__ h_out,
-    int d, int clear_y, const float* __restrict__ y_next) {
+    int d, int clear_y, const float* __restrict__ y_next, const float* __restrict__ y_bias, const float* __restrict__ row_add) {
     __shared__ float scratch[PN_WAVES];
     const long long row = (long long)blockIdx.x * d;
-    float xv[EPT], yv[EPT], wv[EPT], ev[EPT], nv[EPT];
+    float xv[EPT], yv[EPT], wv[EPT], ev[EPT], rv[EPT], nv[EPT];
 #pragma unroll
     for (int k = 0; k < EPT; ++k) {
         const int c = threadIdx.x + k * PN_THREADS;
         const bool in = c < d;
         xv[k] = in ? x[row + c] : 0.f;
         yv[k] = (in && y) ? y[row + c] : 0.f;
+        if (y_bias && in) yv[k] += y_bias[c];
         wv[k] = (in && y) ? w[c] : 0.f;
         ev[k] = (in && extra) ? extra[row + c] : 0.f;
-        nv[k] = (in && h_out) ? w_next[c] : 0.f;
+        rv[k] = (in && row_add) ? row_add[c] : 0.f;
+        nv[k] = (in && w_next) ? w_next[c] : 0.f;
     }
     float inv = 0.f;
     if (y) {
@@ -101,11 +113,20 @@ __global__ __launch_bounds__(PN_THREADS) void post_norm_add_regs_kernel(
             if (clear_y) y[row + c] = y_next ? y_next[c] : 0.f;
         }
         if (extra) v += ev[k];
-        if (y || extra) x[row + c] = v;
+        if (row_add) v += rv[k];
+        if (y || extra || row_add) x[row + c] = v;
         xv[k] = v;
         ss2 = fmaf(v, v, ss2);
     }
     if (!h_out) return;
+    if (!w_next) {
+#pragma unroll
+        for (int k = 0; k < EPT; ++k) {
+            const int c = threadIdx.x + k * PN_THREADS;
+            if (c < d) h_out[row + c] = from_f32<T>(xv[k]);
+        }
+        return;
+    }
     ss2 = block_sum<PN_WAVES>(ss2, scratch);
     const float inv2 = 1.0f / sqrtf(ss2 / (float)d + eps_next);
 #pragma unroll
@@ -220,14 +241,15 @@ TUFF_EXPORT int tuff_scale_add_layer_norm(float* x, float* y, const float* ls, c
 }
 
 // x float32 [T][d] in place; y float32 [T][d] or null; w float32 [d] (with y); extra float32 [T][d] or null;
-// w_next float32 [d] and h_out [T][d] of type out_dt, or both null; y_next float32 [d] or null (with clear_y).
+// h_out [T][d] of type out_dt or null, with w_next float32 [d] or null (no norm); y_next float32 [d] or null (with clear_y);
+// y_bias float32 [d] (with y) and row_add float32 [d], each or null.
 TUFF_EXPORT int tuff_post_norm_add(float* x, float* y, const float* w, float eps, float mult, const float* extra,
                                    const float* w_next, float eps_next, void* h_out, int out_dt, int n_tokens, int d,
-                                   int clear_y, const float* y_next, hipStream_t stream) {
+                                   int clear_y, const float* y_next, const float* y_bias, const float* row_add, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
-    if (d <= 0 || (y && !w) || ((w_next == nullptr) != (h_out == nullptr))) return -2;
+    if (d <= 0 || (y && !w) || (w_next && !h_out) || (y_bias && !y)) return -2;
     dim3 grid(n_tokens), block(PN_THREADS);
-#define LAUNCH(KERN, T) hipLaunchKernelGGL(KERN, grid, block, 0, stream, x, y, w, eps, mult, extra, w_next, eps_next, (T*)h_out, d, clear_y, y_next)
+#define LAUNCH(KERN, T) hipLaunchKernelGGL(KERN, grid, block, 0, stream, x, y, w, eps, mult, extra, w_next, eps_next, (T*)h_out, d, clear_y, y_next, y_bias, row_add)
     if (d <= PN_THREADS * 8) {
         if (out_dt == DT_F32) LAUNCH((post_norm_add_regs_kernel<float, 8>), float); else LAUNCH((post_norm_add_regs_kernel<bf16_t, 8>), bf16_t);
     } else if (d <= PN_THREADS * 32) {

@@ -287,6 +287,125 @@ __global__ void rope_table_kernel(const float* __restrict__ inv_freq, int n_freq
     out[((long long)p * 2 + 1) * n_freq + j] = sinf(a);
 }
 
+// After a q/k/v projection that leaves its float32 sums: biases, half-split rotation of q and k over their first rotary_dim
+// channels, and the write of k and v into the paged cache, for values of any width and for cache rows that hold `maps` keys
+// side by side (key head i is part i % maps of kv head i / maps's row).  Two kinds of workgroups in one launch:
+//  * q and k: a thread takes VEC rotated pairs (or VEC channels that pass) of one token and walks a share of the token's
+//    heads with them, so cosines and sines are computed once for all of these heads;
+//  * v: a workgroup takes sixteen consecutive tokens and 64 channels of one kv head through LDS and writes, for every
+//    channel, the sixteen positions in one run where the tokens fill sixteen slots from a multiple of sixteen, else one by one.
+constexpr int RW_CH = 64;                            // channels of a v workgroup
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void rotate_write_kernel(
+    const float* __restrict__ qkv, const float* __restrict__ bias, T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache,
+    const float* __restrict__ inv_freq, int rotary_dim, const int* __restrict__ positions, const int* __restrict__ slot_mapping,
+    int n_tokens, int H, int Hk, int hd, int maps, int vd, int page_size, int shares, int qk_blocks,
+    const float* __restrict__ angles, int n_angles) {
+    const int tid = threadIdx.x;
+    const int G = Hk / maps;
+    const long long width = (long long)(H + Hk) * hd + (long long)G * vd;
+    if ((int)blockIdx.x < qk_blocks) {
+        const int half = rotary_dim / 2, turning = half / VEC, units = turning + (hd - rotary_dim) / VEC;
+        const long long idx = (long long)blockIdx.x * 256 + tid;
+        const int unit = (int)(idx % units);
+        const long long item = idx / units;
+        const int t = (int)(item / shares), share = (int)(item % shares);
+        if (t >= n_tokens) return;
+        const bool turns = unit < turning;
+        const int j = turns ? unit * VEC : rotary_dim + (unit - turning) * VEC;
+        float rc[VEC], rs[VEC];
+        if (turns) {
+            const int p = positions[t];
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) {
+                if (p < n_angles) {                  // from the table: the same bits, without the two functions
+                    rc[e] = angles[((long long)p * 2) * half + j + e];
+                    rs[e] = angles[((long long)p * 2 + 1) * half + j + e];
+                } else {
+                    const float a = (float)p * inv_freq[j + e];
+                    rc[e] = cosf(a);
+                    rs[e] = sinf(a);
+                }
+            }
+        }
+        const long long slot = k_cache ? slot_mapping[t] : -1;
+        const long long page = slot / page_size, off = slot % page_size;
+        const int heads = slot >= 0 ? H + Hk : H;    // (without a cache to write the keys are not looked at)
+        const int per = (H + Hk + shares - 1) / shares;
+        typedef float vec __attribute__((ext_vector_type(VEC)));
+        typedef T out_vec __attribute__((ext_vector_type(VEC)));
+        for (int head = share * per; head < min(heads, (share + 1) * per); ++head) {
+            const float* src = qkv + t * width + (long long)head * hd + j;
+            const float* b = bias ? bias + (long long)head * hd + j : nullptr;
+            T* dst;
+            if (head < H) dst = q_out + ((long long)t * H + head) * hd + j;
+            else {
+                const int kh = head - H;
+                dst = k_cache + ((page * G + kh / maps) * page_size + off) * (maps * hd) + (kh % maps) * hd + j;
+            }
+            vec u = *(const vec*)src;
+            if (b) u += *(const vec*)b;
+            if (!turns) {
+                out_vec o;
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) o[e] = from_f32<T>(u[e]);
+                *(out_vec*)dst = o;
+                continue;
+            }
+            vec v = *(const vec*)(src + half);
+            if (b) v += *(const vec*)(b + half);
+            out_vec o0, o1;
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) {
+                o0[e] = from_f32<T>(u[e] * rc[e] - v[e] * rs[e]);
+                o1[e] = from_f32<T>(u[e] * rs[e] + v[e] * rc[e]);
+            }
+            *(out_vec*)dst = o0;
+            *(out_vec*)(dst + half) = o1;
+        }
+        return;
+    }
+    __shared__ T vt[P64_TOKENS][RW_CH + 2];
+    __shared__ int slots[P64_TOKENS];
+    const int tiles = (vd + RW_CH - 1) / RW_CH;
+    const int vb = (int)blockIdx.x - qk_blocks;
+    const int c0 = (vb % tiles) * RW_CH, kvh = (vb / tiles) % G, t0 = vb / (tiles * G) * P64_TOKENS;
+    const int n_here = min(P64_TOKENS, n_tokens - t0), n_ch = min(RW_CH, vd - c0);
+    const long long col = (long long)(H + Hk) * hd + (long long)kvh * vd + c0;
+    for (int i = tid / RW_CH; i < n_here; i += 256 / RW_CH) {
+        const int c = tid % RW_CH;
+        if (c < n_ch) vt[i][c] = from_f32<T>(qkv[(t0 + i) * width + col + c] + (bias ? bias[col + c] : 0.f));
+    }
+    if (tid < P64_TOKENS) slots[tid] = tid < n_here ? slot_mapping[t0 + tid] : -1;
+    __syncthreads();
+    const int s0 = slots[0];
+    bool run = n_here == P64_TOKENS && s0 >= 0 && s0 % 16 == 0 && page_size % 16 == 0;
+#pragma unroll
+    for (int i = 1; i < P64_TOKENS; ++i) run = run && slots[i] == s0 + i;
+    if (run) {
+        if (tid < n_ch) {
+            const long long page = s0 / page_size, off = s0 % page_size;
+            T* dst = v_cache + ((page * G + kvh) * vd + c0 + tid) * page_size + off;
+            T vals[P64_TOKENS];
+#pragma unroll
+            for (int i = 0; i < P64_TOKENS; ++i) vals[i] = vt[i][tid];
+            constexpr int PIECES = P64_TOKENS * (int)sizeof(T) / 16;
+#pragma unroll
+            for (int q = 0; q < PIECES; ++q) ((uint4*)dst)[q] = ((const uint4*)vals)[q];
+        }
+    } else {
+        const int ch = tid % RW_CH;
+        if (ch < n_ch)
+            for (int i = tid / RW_CH; i < n_here; i += 256 / RW_CH) {
+                const long long slot = slots[i];
+                if (slot < 0) continue;
+                const long long page = slot / page_size, off = slot % page_size;
+                v_cache[((page * G + kvh) * vd + c0 + ch) * page_size + off] = vt[i][ch];
+            }
+    }
+}
+
 // Copies already encoded k and v rows [T, Hkv, hd] into the paged cache.
 template <typename T>
 __global__ __launch_bounds__(WAVE) void kv_write_kernel(const T* __restrict__ k, const T* __restrict__ v,
@@ -377,5 +496,35 @@ TUFF_EXPORT int tuff_rope_table(const float* inv_freq, int n_freq, int n_pos, fl
     if (n_pos <= 0 || n_freq <= 0) return 0;
     const long long n = (long long)n_pos * n_freq;
     hipLaunchKernelGGL(rope_table_kernel, dim3((unsigned)ceil_div_ll(n, 256)), dim3(256), 0, stream, inv_freq, n_freq, n_pos, out);
+    return launch_status();
+}
+
+// qkv float32 [T][(H + Hk) hd + (Hk / maps) vd]: H query heads and Hk key heads of hd channels, then Hk / maps value heads of vd;
+// bias float32 of a row's width, or null.  q_out [T][H hd] and the caches (K [page][kv head][offset][maps hd], V [page][kv head]
+// [vd][offset]; null: nothing is written) of type dt.  inv_freq float32 [rotary_dim / 2] (null with rotary_dim 0); angles as
+// tuff_rope_table makes them, or null.
+TUFF_EXPORT int tuff_qkv_rotate_write(const float* qkv, const float* bias, void* q_out, void* k_cache, void* v_cache, int dt,
+                                      const float* inv_freq, int rotary_dim, const int* positions, const int* slot_mapping, int n_tokens,
+                                      int H, int Hk, int hd, int maps, int vd, int page_size, const float* angles, int n_angles,
+                                      hipStream_t stream) {
+    if (n_tokens <= 0) return 0;
+    if (H < 1 || Hk < 1 || maps < 1 || Hk % maps || hd < 1 || vd < 1 || rotary_dim < 0 || rotary_dim > hd || rotary_dim % 2 || page_size < 1) return -2;
+    if ((rotary_dim > 0 && !inv_freq) || ((k_cache == nullptr) != (v_cache == nullptr)) || (k_cache && !slot_mapping)) return -2;
+    if (!angles) n_angles = 0;
+    const long long width = (long long)(H + Hk) * hd + (long long)(Hk / maps) * vd;
+    const bool four = (rotary_dim / 2) % 4 == 0 && hd % 4 == 0 && width % 4 == 0 && (uintptr_t)bias % 16 == 0;
+    const int units = four ? rotary_dim / 8 + (hd - rotary_dim) / 4 : rotary_dim / 2 + (hd - rotary_dim);
+    // shares of a token's heads: enough threads for the chip, whole heads each
+    int shares = 1;
+    while (shares < H + Hk && (long long)n_tokens * shares * units < 262144) shares *= 2;
+    shares = min(shares, H + Hk);
+    const long long qk = ceil_div_ll((long long)n_tokens * shares * units, 256);
+    const long long vb = k_cache ? (long long)ceil_div(n_tokens, P64_TOKENS) * (Hk / maps) * ceil_div(vd, RW_CH) : 0;
+    if (qk + vb > 0x7fffffffll) return -2;
+#define LAUNCH(T, V) hipLaunchKernelGGL((rotate_write_kernel<T, V>), dim3((unsigned)(qk + vb)), dim3(256), 0, stream, qkv, bias, (T*)q_out, \
+        (T*)k_cache, (T*)v_cache, inv_freq, rotary_dim, positions, slot_mapping, n_tokens, H, Hk, hd, maps, vd, page_size, shares, (int)qk, angles, n_angles)
+    if (dt == DT_F32) { if (four) LAUNCH(float, 4); else LAUNCH(float, 1); }
+    else { if (four) LAUNCH(bf16_t, 4); else LAUNCH(bf16_t, 1); }
+#undef LAUNCH
     return launch_status();
 }

@@ -11,6 +11,7 @@ import torch
 
 from ..csrc import ops
 from ..parts.base import Block, FixedState, Norm, PagedKV, Runtime, WeightDecl, cache_specs_of
+from ..parts.block import PLAIN_ROWS
 from ..parts.norm import RMSNorm
 
 
@@ -20,6 +21,7 @@ class LayerRun:
     cache: Optional[int] = None     # cache entry this run uses (default: one of its own)
     writes: bool = True             # False: only reads the entry, which an earlier run writes
     reinject: bool = False          # True: the embedding (as it entered the first run) is added to x before this run
+    enter: Optional[int] = None     # the number of the pass that begins with this run (DecoderModel's entry)
 
 
 class _Head:
@@ -32,7 +34,7 @@ _HEAD = _Head()
 
 def _any_window(spec):
     """A declaration without its window: runs that share an entry may read windows of different widths."""
-    return dataclasses.replace(spec, window=None) if isinstance(spec, PagedKV) else spec
+    return dataclasses.replace(spec, window=None, keep_first=0) if isinstance(spec, PagedKV) else spec
 
 
 class DecoderModel:
@@ -41,7 +43,7 @@ class DecoderModel:
                  schedule: Optional[list[LayerRun]] = None, max_positions: Optional[int] = None,
                  eos_token_id: Optional[int] = None, embedding_scale: float = 1.0,
                  logit_scale: float = 1.0, logit_softcap: Optional[float] = None, pad_hidden: bool = False,
-                 streams: Optional[int] = None, depth_average: Optional[list[WeightDecl]] = None):
+                 streams: Optional[int] = None, depth_average: Optional[list[WeightDecl]] = None, entry=None):
         """head=None: the head is the embedding (tied), as the reference does when the file has
         no output matrix (src/lfm25_model.c:128-131).
         embedding_scale: the embedding rows are multiplied by it on their way into the residual stream.
@@ -52,7 +54,9 @@ class DecoderModel:
         streams: the model keeps that many residual streams [S, T, d], all equal to the embedding at the start
         and summed before the final norm; its blocks are then all of a kind that takes them (multi_stream).
         depth_average: one weight a run, [i + 2] for run i: with X_0 the embedding and X_(i+1) what run i makes of its
-        input, what goes on after run i is the sum of weight[j] X_j, j = 0 .. i + 1."""
+        input, what goes on after run i is the sum of weight[j] X_j, j = 0 .. i + 1.
+        entry: a parts.loop.PassEntry; before a run with `enter` = t the stream becomes what the entry makes of it, of the
+        embedding and of t (blocks of the kind that hand each other their first input only)."""
         self.pad_hidden = bool(pad_hidden)
         self.streams = None if streams is None else int(streams)
         if self.streams is not None and (self.streams < 1 or not all(getattr(b, "multi_stream", False) for b in blocks)):
@@ -69,6 +73,15 @@ class DecoderModel:
         #: every block hands the next one its first normed input (Block.carries_norm): the kernel that adds a block's
         #: last output into the stream also reads the stream for whoever comes next
         self.carries = bool(blocks) and all(getattr(b, "carries_norm", False) for b in blocks)
+        runs_ = schedule if schedule is not None else []
+        self.entry = entry
+        if entry is None and any(r.enter is not None for r in runs_):
+            raise ValueError("a run begins a pass of a model without an entry")
+        if entry is not None:
+            if not self.carries or not all(getattr(b, "hands_plain_rows", False) for b in blocks):
+                raise ValueError("passes with an entry need blocks that hand on the stream itself")
+            if any(r.enter is not None and (r.reinject or not 0 <= r.enter < entry.times) for r in runs_):
+                raise ValueError(f"a run begins a pass outside 0 .. {entry.times - 1}, or takes the embedding twice")
         #: debugging aid: called as on_layer(run index, x [T, d] or xs [S, T, d]) after every layer run; while it
         #: is set no step is recorded into a graph
         self.on_layer = None
@@ -91,7 +104,7 @@ class DecoderModel:
                     next_id += 1
                 cache = next_id
                 used.add(cache)
-            self.schedule.append(LayerRun(r.block, cache, r.writes, r.reinject))
+            self.schedule.append(LayerRun(r.block, cache, r.writes, r.reinject, r.enter))
         # Every cache entry has exactly one writer, which comes before its readers.  A run's entry is named
         # by LayerRun.cache; a mixer that declares several things to keep has the entries (cache, 0),
         # (cache, 1), ... in the order of its declarations.
@@ -123,8 +136,11 @@ class DecoderModel:
                 # the entry keeps what the widest window of its runs reads
                 for e, spec in zip(ids, specs):
                     kept = self.cache_specs[e]
-                    if kept.window is not None and (spec.window is None or spec.window > kept.window):
-                        self.cache_specs[e] = dataclasses.replace(kept, window=spec.window)
+                    if kept.window is None:
+                        continue
+                    window = None if spec.window is None else max(kept.window, spec.window)
+                    keep = 0 if window is None else max(kept.keep_first, spec.keep_first)
+                    self.cache_specs[e] = dataclasses.replace(kept, window=window, keep_first=keep)
             self._run_entries.append((several, ids))
         self.embedding: Optional[torch.Tensor] = None
         self.head: Optional[torch.Tensor] = None
@@ -132,8 +148,15 @@ class DecoderModel:
     # ------------------------------------------------------------------ description
     def weight_decls(self) -> list[WeightDecl]:
         decls = [self.embedding_decl]
+        shared: dict = {}                        # tensors several parts read, once each
         for b in self.blocks:
             decls += b.weight_decls()
+            for d in b.shared_decls():
+                if shared.setdefault(d.name, d) != d:
+                    raise ValueError(f"two parts declare the shared tensor '{d.name}' differently: {shared[d.name]} and {d}")
+        decls += list(shared.values())
+        if self.entry is not None:
+            decls += self.entry.weight_decls()
         decls += self.final_norm.weight_decls()
         decls += self.depth_decls or []
         if self.head_decl is not None:
@@ -150,7 +173,7 @@ class DecoderModel:
         mods = ["elementwise"] + (["depth"] if self.depth_decls is not None else [])
         for b in self.blocks:
             mods += b.kernel_modules()
-        mods += self.final_norm.kernel_modules()
+        mods += self.final_norm.kernel_modules() + (self.entry.kernel_modules() if self.entry is not None else [])
         return sorted(set(mods))
 
     def token_inputs(self) -> tuple:
@@ -181,6 +204,8 @@ class DecoderModel:
         for b in self.blocks:
             b.bind(weights, rt)
         self.final_norm.bind(weights, rt)
+        if self.entry is not None:
+            self.entry.bind(weights, rt)
         self._head_cast: Optional[torch.Tensor] = None
         if self.depth_decls is not None:
             self.depth_w = [weights[w.name].float().contiguous() for w in self.depth_decls]
@@ -276,10 +301,18 @@ class DecoderModel:
         last = len(self.schedule) - 1
         y = torch.empty(ctx.T, self.hidden_size, dtype=torch.float32, device=self.rt.device)
         ops.fill_u32(y, 0)
-        carry = None
+        carry = z0 = None
         for i, run in enumerate(self.schedule):
             block = self.blocks[run.block]
             nxt = self.schedule[i + 1] if i < last else None
+            if run.enter is not None:
+                if z0 is None:                                  # (the first pass of the step)
+                    rows = self.rt.empty(ctx.T, self.hidden_size)
+                    ops.embed_rows(self.embedding, ctx.tokens, rows, self.embedding_scale)
+                    z0 = self.entry.embedding_part(rows)
+                    if carry is None:                           # nothing ran before: the stream is the embedding
+                        carry = rows
+                x, carry = self.entry.forward(carry, z0, run.enter, block.first_read())
             extra = x0 if nxt is not None and nxt.reinject else None
             if run.reinject and carry is None:
                 ops.post_norm_add(x, extra=x0)              # (nobody before this run could add it)
@@ -289,7 +322,7 @@ class DecoderModel:
                 self.on_layer(i, x)
                 carry = None
                 continue
-            read = self.blocks[nxt.block].first_read() if nxt is not None else None
+            read = None if nxt is None else PLAIN_ROWS if nxt.enter is not None else self.blocks[nxt.block].first_read()
             carry = block.forward(x, ctx, self._views_of(i, cache_views), run.writes, carry=carry, next_read=read, y=y, extra=extra)
             if self.on_layer is not None:
                 self.on_layer(i, x)

@@ -83,6 +83,9 @@ def _register_builtin() -> None:
     from ..config.kisutar import KisutarConfig
     from .kisutar import build_kisutar
     register_architecture(KisutarConfig.architecture, KisutarConfig, build_kisutar)
+    from ..config.tobilorn import TobilornConfig
+    from .tobilorn import build_tobilorn
+    register_architecture(TobilornConfig.architecture, TobilornConfig, build_tobilorn)
 
 
 _register_builtin()

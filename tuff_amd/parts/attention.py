@@ -10,7 +10,8 @@ score of query i and key j, slope_h = 2^(-span (h + 1) / H).  Further options: b
 logarithmic distance penalty r1_h ln(1 + r2_h (i - j)) with learned r1, r2 per head; the heads' softmax
 weights mixed by a learned [H, H] matrix, p'_h = sum_g talk[h, g] p_g, head h applying p'_h to the values of
 its own kv head; a short causal convolution per channel on q, k and v right after the projection (its last
-taps - 1 inputs are state of the request); a gate per head, sigmoid(W_g h)_h, on the head's output.
+taps - 1 inputs are state of the request); a gate per head, sigmoid(W_g h)_h, on the head's output; a window that keeps
+the sequence's first tokens visible.  DifferentialAttentionMixer: two softmax maps a head, the second taken off the first.
 Reference: src/lfm25_engine.c:386-405, src/lfm25_gpu.cu:420-485, :506-558.
 """
 from __future__ import annotations
@@ -32,7 +33,9 @@ class PagedAttention:
     grouped heads and optional sinks.  It reads the mixer's H, Hkv, hd, vd, window, scale, sinks, slopes and, where
     the mixer has them, log_distance ((r1, r2): the penalty r1_h ln(1 + r2_h (i - j))) and talk (a matrix that mixes
     the heads' softmax weights: o is then float32 [T, H * Hkv * vd], every head's weights on every kv head's values,
-    from which ops.head_mix_gate forms the mixed heads)."""
+    from which ops.head_mix_gate forms the mixed heads), keep_first (a window's tokens also see the sequence's first
+    keep_first keys) and combine ((lambda, eps, coef): differential attention; H counts softmax maps, two a head, hd is the
+    width of a key row that holds both maps' keys, q [T, H * hd / 2], and o [T, H / 2 * vd] the combined and normed heads)."""
 
     @staticmethod
     def _upload(array, device):
@@ -79,6 +82,8 @@ class PagedAttention:
         for all heads, and mix and gate the heads themselves."""
         special = (getattr(self, "log_distance", None) is not None or getattr(self, "talk", None) is not None
                    or getattr(self, "exact_weights", False))
+        # (those kernels know neither kept first keys nor several maps a head)
+        special = special and not getattr(self, "keep_first", 0) and getattr(self, "combine", None) is None
         return (special and ctx.max_q_len == 1
                 and ops.attention_decode_exact_supported(dtype, self.H, self.hd, self.vd, page_size))
 
@@ -86,13 +91,17 @@ class PagedAttention:
         G = self.H // self.Hkv
         log_distance, talk = getattr(self, "log_distance", None), getattr(self, "talk", None)
         exact = getattr(self, "exact_weights", False)
+        keep, combine = getattr(self, "keep_first", 0), getattr(self, "combine", None)
+        if combine is not None:
+            self._attend_maps(q, o, ctx, cache, g, keep, combine)
+            return
         if (exact and log_distance is None and talk is None and gates is None and ctx.max_q_len == 1
                 and ops.attention_single_supported(q.dtype, self.hd, self.vd, cache.page_size)):
             # single tokens with float32 weights on the matrix cores
             ops.attention_single(q, cache.k, cache.v, o, block_table=g.block_table, req_of_token=ctx.req_of_token,
                                  positions=ctx.positions, H=self.H, Hkv=self.Hkv, hd=self.hd, vd=self.vd, page_size=cache.page_size,
                                  max_ctx_len=ctx.max_ctx_len, window=self.window or 0, scale=self.scale, sinks=self.sinks,
-                                 slopes=self.slopes)
+                                 slopes=self.slopes, keep_first=keep)
             return
         if self._single_tokens_exact(q.dtype, ctx, cache.page_size):
             ops.attention_decode_exact(q, cache.k, cache.v, o, block_table=g.block_table, req_of_token=ctx.req_of_token,
@@ -110,14 +119,14 @@ class PagedAttention:
                                        blocks=self._blocks(ctx, G, nb, q.device, longest_first=True), req_info=ctx.req_info,
                                        H=self.H, Hkv=self.Hkv, hd=self.hd, vd=self.vd, page_size=cache.page_size,
                                        max_ctx_len=ctx.max_ctx_len, window=self.window or 0, scale=self.scale, sinks=self.sinks,
-                                       slopes=self.slopes, log_distance=log_distance, all_values=talk is not None)
+                                       slopes=self.slopes, log_distance=log_distance, all_values=talk is not None, keep_first=keep)
             return
         if log_distance is not None or talk is not None or exact:
             ops.attention_general(q, cache.k, cache.v, o, block_table=g.block_table,
                                   req_of_token=ctx.req_of_token, positions=ctx.positions,
                                   H=self.H, Hkv=self.Hkv, hd=self.hd, page_size=cache.page_size,
                                   window=self.window or 0, scale=self.scale, vd=self.vd, sinks=self.sinks, slopes=self.slopes,
-                                  log_distance=log_distance, all_values=talk is not None)
+                                  log_distance=log_distance, all_values=talk is not None, keep_first=keep)
             return
         if self.vd == self.hd and ops.attention_mfma_supported(q.dtype, self.hd, cache.page_size):
             common = dict(block_table=g.block_table, req_info=ctx.req_info, H=self.H, Hkv=self.Hkv, hd=self.hd,
@@ -148,6 +157,25 @@ class PagedAttention:
                               H=self.H, Hkv=self.Hkv, hd=self.hd, page_size=cache.page_size,
                               window=self.window or 0, scale=self.scale, vd=self.vd, sinks=self.sinks, slopes=self.slopes)
 
+    def _attend_maps(self, q, o, ctx, cache, g, keep, combine) -> None:
+        """Two softmax maps a head over one kv head's values (see `combine` above)."""
+        dim, ps = self.hd // 2, cache.page_size
+        common = dict(block_table=g.block_table, Hkv=self.Hkv, vd=self.vd, page_size=ps, window=self.window or 0, scale=self.scale,
+                      keep_first=keep)
+        if ctx.max_q_len > 1 and ops.attention_prefill_diff_supported(q.dtype, dim, self.vd, ps):
+            nb = ops.attention_prefill_diff_block_columns() // 16
+            blocks = self._blocks(ctx, self.H // 2 // self.Hkv, nb, q.device, longest_first=True)
+            ops.attention_prefill_diff(q, cache.k, cache.v, o, blocks=blocks, req_info=ctx.req_info, heads=self.H // 2, dim=dim,
+                                       max_ctx_len=ctx.max_ctx_len, combine=combine, **common)
+            return
+        common.update(req_of_token=ctx.req_of_token, positions=ctx.positions, H=self.H, hd=self.hd)
+        if ctx.max_q_len == 1 and dim % 8 == 0 and ops.attention_single_supported(q.dtype, self.hd, self.vd, ps):
+            ops.attention_single(q, cache.k, cache.v, o, max_ctx_len=ctx.max_ctx_len, combine=combine, **common)
+            return
+        maps = torch.empty(q.shape[0], self.H * self.vd, dtype=torch.float32, device=q.device)
+        ops.attention_general(q, cache.k, cache.v, maps, maps=2, **common)
+        ops.diff_combine(maps, o, H=self.H // 2, vd=self.vd, combine=combine)
+
 
 @MIXERS.register("attention")
 class AttentionMixer(Mixer, PagedAttention):
@@ -159,7 +187,7 @@ class AttentionMixer(Mixer, PagedAttention):
                  position: Optional[PositionEncoding] = None, window: Optional[int] = None,
                  scale: Optional[float] = None, aliases: Optional[dict[str, tuple]] = None,
                  value_dim: Optional[int] = None, slope_span: Optional[float] = None, conv_taps: Optional[int] = None,
-                 exact_weights: bool = False):
+                 exact_weights: bool = False, keep_first: int = 0):
         """names: checkpoint names of 'q', 'k', 'v', 'o' and, with qk_norm_eps, 'q_norm', 'k_norm' (without these
         two names the norm has no weight: q and k are divided by their root mean square over the head); with a
         'sink' among them the heads have sinks.  value_dim: width of a value head (default: head_dim).
@@ -169,8 +197,13 @@ class AttentionMixer(Mixer, PagedAttention):
         gate per head; with conv_taps, 'q.conv', 'k.conv', 'v.conv' [channels, taps] the convolutions' taps (one tap: a
         factor per channel and no state).
         exact_weights: the softmax weights keep float32's precision where they meet the values, also with bfloat16
-        activations (the kernels that round them to bfloat16 for the matrix cores are not used)."""
+        activations (the kernels that round them to bfloat16 for the matrix cores are not used).
+        keep_first (with a window and exact_weights): every token also sees the sequence's first keep_first tokens, in their
+        true places."""
         self.exact_weights = bool(exact_weights)
+        self.keep_first = int(keep_first) if window else 0
+        if self.keep_first and not self.exact_weights:
+            raise ValueError("first tokens that stay visible go with exact_weights (the other kernels know windows only)")
         if num_heads % num_kv_heads:
             raise ValueError(f"heads {num_heads} must be a multiple of kv heads {num_kv_heads}")
         if head_dim > 256:
@@ -247,7 +280,7 @@ class AttentionMixer(Mixer, PagedAttention):
         return self.position.token_inputs() if self.position is not None else []
 
     def cache_spec(self):
-        kv = PagedKV(self.Hkv, self.hd, self.window, value_dim=None if self.vd == self.hd else self.vd)
+        kv = PagedKV(self.Hkv, self.hd, self.window, value_dim=None if self.vd == self.hd else self.vd, keep_first=self.keep_first)
         # with a convolution: its last taps - 1 inputs, then the keys and values
         return (FixedState((self.K - 1, self.C)), kv) if self.K > 1 else kv
 
@@ -361,3 +394,107 @@ class AttentionMixer(Mixer, PagedAttention):
             heads = self.rt.empty(T, H * vd)
             ops.head_mix_gate(o, heads, H=H, Hkv=Hkv, vd=vd, talk=self.talk, gates=gates)
         self.out.forward(heads, accumulate_into=residual, next_norm=next_norm)
+
+
+@MIXERS.register("differential_attention")
+class DifferentialAttentionMixer(Mixer, PagedAttention):
+    """Differential attention over the paged cache: a head has two softmax maps over the same values, each with queries and
+    keys of its own (W_q [H 2 dim, d], W_k [Hkv 2 dim, d], a head's maps side by side); with a1, a2 the maps' outputs and one
+    number a layer, lambda = exp(sum lq1 lk1) - exp(sum lq2 lk2) + diff,
+        v = a1 - lambda a2,   out_head = v / sqrt(mean(v^2) + eps) (1 - diff)     (the mean over the head's vdim channels)
+    and W_o on the heads.  Scores are scaled by `scale`; optional biases of the four projections, half-split rotation of each
+    map's q and k, a window (a token and the window - 1 before it) with or without the sequence's first keep_first tokens.
+
+    A kv head's cache row holds both maps' keys, 2 dim channels, and its values once: the attention kernels read a row once
+    for both maps and combine them.  Between the projection and the cache one kernel takes the product's float32 sums, adds
+    the biases, rotates and writes."""
+    accepts_pending_norm = True
+    adds_once_through_linear = True
+    records_portions = True
+    graph_safe = True
+
+    def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int, *, names: dict[str, str],
+                 scale: float, diff: float, norm_eps: float, position: Optional[PositionEncoding] = None,
+                 window: Optional[int] = None, keep_first: int = 0):
+        """names: checkpoint names of 'q', 'k', 'v', 'o', of 'lq1', 'lk1', 'lq2', 'lk2' [dim] and, for biases, of 'q.b', 'k.b',
+        'v.b', 'o.b'.  position: a rotary encoding in the half-split form, or None."""
+        if num_heads % num_kv_heads:
+            raise ValueError(f"heads {num_heads} must be a multiple of kv heads {num_kv_heads}")
+        if 2 * head_dim > ops.ATTN_GENERAL_MAX_DIM or value_dim > ops.ATTN_GENERAL_MAX_DIM:
+            raise ValueError(f"head sizes {head_dim} and {value_dim}: a key row of both maps and a value are at most "
+                             f"{ops.ATTN_GENERAL_MAX_DIM} channels wide")
+        if position is not None:
+            tables = position.rotary_tables()
+            if tables is None or tables[2]:
+                raise ValueError("differential attention takes a half-split rotary encoding or none")
+        self.d, self.heads, self.dim = int(hidden_size), int(num_heads), int(head_dim)
+        # what PagedAttention reads: H counts maps, hd is a key row's width
+        self.H, self.Hkv, self.hd, self.vd = 2 * self.heads, int(num_kv_heads), 2 * self.dim, int(value_dim)
+        self.window = int(window) if window else None
+        self.keep_first = int(keep_first) if window else 0
+        self.scale, self.diff, self.eps = float(scale), float(diff), float(norm_eps)
+        self.sinks = self.slopes = None
+        self.exact_weights = True
+        self.combine = None                    # bound: (lambda, eps, 1 - diff)
+        self.position = position
+        self.names = dict(names)
+        self.has_bias = "q.b" in self.names
+        self.outs = [self.H * self.dim, 2 * self.Hkv * self.dim, self.Hkv * self.vd]
+        # (the biases ride in the kernels that follow the products)
+        self.qkv = Linear([names["q"], names["k"], names["v"]], self.d, self.outs)
+        self.out = Linear(names["o"], self.heads * self.vd, self.d)
+        self.qkv_bias = None
+        #: float32 [d] once bound, or None: what the mixer adds to every row of its output.  A block that reads the rows the
+        #: mixer added into may add it there and say so (forward(bias_deferred=True))
+        self.output_bias = None
+
+    def weight_decls(self):
+        n = self.names
+        decls = self.qkv.weight_decls() + self.out.weight_decls()
+        if self.has_bias:
+            decls += [WeightDecl(n[k], (w,), "normal") for k, w in zip(("q.b", "k.b", "v.b", "o.b"), self.outs + [self.d])]
+        decls += [WeightDecl(n[k], (self.dim,), "normal") for k in ("lq1", "lk1", "lq2", "lk2")]
+        return decls + (self.position.weight_decls() if self.position is not None else [])
+
+    def kernel_modules(self):
+        return ["rope_kv", "elementwise", "attention", "attention_prefill", "attention_single"]
+
+    def cache_spec(self):
+        return PagedKV(self.Hkv, self.hd, self.window, value_dim=None if self.vd == self.hd else self.vd, keep_first=self.keep_first)
+
+    def bind(self, weights, rt: Runtime):
+        self.rt = rt
+        n = self.names
+        self.qkv.bind(weights, rt)
+        self.out.bind(weights, rt)
+        if self.has_bias:
+            self.qkv_bias = torch.cat([weights[n[k]].float() for k in ("q.b", "k.b", "v.b")]).contiguous()
+            self.output_bias = weights[n["o.b"]].float().contiguous()
+        l1, l2 = (float((weights[n["lq" + i]].double() * weights[n["lk" + i]].double()).sum()) for i in ("1", "2"))
+        self.combine = (math.exp(l1) - math.exp(l2) + self.diff, self.eps, 1.0 - self.diff)
+        if self.position is not None:
+            self.position.bind(weights, rt)
+
+    def forward(self, h, ctx, cache, residual, write_cache: bool = True, next_norm=None, bias_deferred: bool = False) -> None:
+        qkv = self.qkv.forward(h, out_dtype=torch.float32)
+        T = qkv.shape[0]
+        q = self.rt.empty(T, self.H * self.dim)
+        o = self.rt.empty(T, self.heads * self.vd)
+        rot = {}
+        if self.position is not None:
+            inv_freq, dims, _ = self.position.rotary_tables()
+            rot = dict(inv_freq=inv_freq, rotary_dim=dims, angles=getattr(self.position, "angle_table", lambda: None)())
+
+        def over_the_cache(ctx):
+            g = ctx.groups[cache.group]
+            wr = dict(k_cache=cache.k, v_cache=cache.v, slot_mapping=g.slot_mapping) if write_cache else {}
+            ops.qkv_rotate_write(qkv, q, H=self.H, Hk=2 * self.Hkv, hd=self.dim, vd=self.vd, maps=2, bias=self.qkv_bias,
+                                 positions=ctx.positions, page_size=cache.page_size, **rot, **wr)
+            self.attend(q, o, ctx, cache, g)
+
+        ctx.run_eagerly(over_the_cache)
+        if self.output_bias is None or bias_deferred:
+            self.out.forward(o, accumulate_into=residual, next_norm=next_norm)
+            return
+        self.out.forward(o, accumulate_into=residual)            # (the sum is not final before the bias is in)
+        ops.add_bias(residual, self.output_bias)

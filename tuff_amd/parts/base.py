@@ -29,7 +29,8 @@ class WeightDecl:
 @dataclasses.dataclass(frozen=True)
 class PagedKV:
     """Keys and values that grow by one entry a token, kept in pages.  `window`: only the
-    last `window` positions are ever read (None: all).  `value_dim`: the width of a value where
+    last `window` positions are ever read (None: all), and with `keep_first` the sequence's first
+    `keep_first` positions besides.  `value_dim`: the width of a value where
     it is not the keys' (None: head_dim).  `value_rows`: values lie as keys do, a row a position
     ([page, kv_head, offset, value_dim]), instead of transposed within the page ([page, kv_head,
     value_dim, offset], which is what the matrix cores of the framework's own attention kernels
@@ -43,6 +44,7 @@ class PagedKV:
     value_dim: Optional[int] = None
     value_rows: bool = False
     values_in_keys: bool = False
+    keep_first: int = 0
 
     @property
     def v_dim(self) -> int:
@@ -106,6 +108,11 @@ class Part:
     """Base of all parts.  `names` maps the part's own weight names to checkpoint names."""
 
     def weight_decls(self) -> list[WeightDecl]:
+        return []
+
+    def shared_decls(self) -> list[WeightDecl]:
+        """Tensors this part reads that other parts of the model read too (a table with a range of columns for every
+        layer): the model declares each once."""
         return []
 
     def bind(self, weights: dict[str, torch.Tensor], rt: Runtime) -> None:

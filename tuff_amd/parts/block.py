@@ -12,6 +12,7 @@ TokenShiftBlock is the pre-norm layer whose mixer reads each row mixed with the 
 
 SandwichBlock norms a sublayer on both sides:
     x += m * norm1b(mixer(norm1(x)));  x += m * norm2b(ffn(norm2(x)))
+and may take in a vector looked up by the token's id after that (parts.side.TokenSide).
 
 LayerScaleBlock is the pre-norm layer whose sublayers' outputs are scaled per channel before they join the stream:
     x += ls1 * mixer(norm1(x));  x += ls2 * ffn(norm2(x))
@@ -28,6 +29,10 @@ import torch
 from ..csrc import ops
 from .base import BLOCKS, Block, FeedForward, FixedState, Mixer, Norm, Runtime, WeightDecl
 from .norm import LayerNorm, RMSNorm
+
+
+#: a block's next_read where whoever reads next wants the stream itself, without a norm
+PLAIN_ROWS = (None, 0.0)
 
 
 @BLOCKS.register("prenorm")
@@ -225,11 +230,14 @@ class SandwichBlock(Block):
     normed before and after.  ffn None: the mixer's sublayer alone.  The four norms are RMS norms (they run inside
     one kernel, ops.post_norm_add, which norms a sublayer's output, adds it into the stream and reads the next
     sublayer's input with its norm; the next sublayer may be the next block's first, so forward() takes what the
-    block before left (`carry`) and is told who reads next (`next_read`))."""
+    block before left (`carry`) and is told who reads next (`next_read`)).
+
+    side: a parts.side.TokenSide, which adds into x after the last sublayer: x <- x + norm_s(side(x, token))."""
     carries_norm = True
+    hands_plain_rows = True            # next_read may be PLAIN_ROWS
 
     def __init__(self, before1: Norm, mixer: Mixer, after1: Norm, before2: Optional[Norm] = None,
-                 ffn: Optional[FeedForward] = None, after2: Optional[Norm] = None, *, mult: float = 1.0):
+                 ffn: Optional[FeedForward] = None, after2: Optional[Norm] = None, *, mult: float = 1.0, side=None):
         if not ((before2 is None) == (ffn is None) == (after2 is None)):
             raise ValueError("before2, ffn and after2 go together")
         for n in (before1, after1, before2, after2):
@@ -237,10 +245,13 @@ class SandwichBlock(Block):
                 raise ValueError("the norms of a sandwich block are RMS norms (they run inside the block's kernel)")
         self.before1, self.mixer, self.after1 = before1, mixer, after1
         self.before2, self.ffn, self.after2 = before2, ffn, after2
-        self.mult = float(mult)
+        self.mult, self.side = float(mult), side
 
     def _parts(self):
-        return [p for p in (self.before1, self.mixer, self.after1, self.before2, self.ffn, self.after2) if p is not None]
+        return [p for p in (self.before1, self.mixer, self.after1, self.before2, self.ffn, self.after2, self.side) if p is not None]
+
+    def shared_decls(self):
+        return [d for p in self._parts() for d in p.shared_decls()]
 
     @property
     def graph_safe(self):
@@ -271,34 +282,47 @@ class SandwichBlock(Block):
     def forward(self, x, ctx, cache, write_cache: bool = True, carry=None, next_read=None, y=None, extra=None):
         """x float32 [T, d], in place.  carry: before1(x) where the block before left it (None: computed here).
         next_read: (norm weight, eps) of whoever reads x next; that norm of the new x is returned (None: nothing is
-        read and None returned).  y: float32 [T, d] of zeros that the sublayers add into (left zero again); None:
-        made here.  extra: float32 [T, d] that joins x after the block's last sublayer, before next_read's norm."""
+        read and None returned; PLAIN_ROWS: x itself in the compute type).  y: float32 [T, d] of zeros that the sublayers add
+        into (left zero again); None: made here.  extra: float32 [T, d] that joins x after everything the block adds,
+        before next_read's norm."""
         T, d = x.shape
         if carry is None:
             carry = self.before1.forward(x)
         if y is None:
             y = torch.empty(T, d, dtype=torch.float32, device=x.device)
             ops.fill_u32(y, 0)
+        if self.side is None:
+            return self._sublayers(x, y, ctx, cache, write_cache, carry, next_read, extra)
+        rows = self._sublayers(x, y, ctx, cache, write_cache, carry, PLAIN_ROWS, None)
+        self.side.forward(rows, ctx, y)
+        return self._join(x, y, self.side.norm, next_read, extra, mult=1.0)
+
+    def _sublayers(self, x, y, ctx, cache, write_cache, carry, next_read, extra):
         kw = {"next_norm": None} if self.mixer.adds_once_through_linear else {}
+        # (a mixer that adds a bias to its output: the kernel that reads y adds it)
+        out_bias = getattr(self.mixer, "output_bias", None)
+        if out_bias is not None:
+            kw["bias_deferred"] = True
         self.mixer.forward(carry, ctx, cache, y, write_cache, **kw)
         if self.ffn is None:
-            return self._join(x, y, self.after1, next_read, extra)
+            return self._join(x, y, self.after1, next_read, extra, y_bias=out_bias)
         # (a feed-forward that adds a bias to its output: the kernel that clears y leaves the bias there instead)
         bias = getattr(self.ffn, "output_bias", None)
-        h = self._join(x, y, self.after1, (self.before2.weight_f32, self.before2.eps), None, y_next=bias)
+        h = self._join(x, y, self.after1, (self.before2.weight_f32, self.before2.eps), None, y_next=bias, y_bias=out_bias)
         kw = {"next_norm": None} if self.ffn.adds_once_through_linear else {}
         if bias is not None:
             kw["bias_preloaded"] = True
         self.ffn.forward(h, ctx, y, **kw)
         return self._join(x, y, self.after2, next_read, extra)
 
-    def _join(self, x, y, after, read, extra, y_next=None):
+    def _join(self, x, y, after, read, extra, y_next=None, y_bias=None, mult=None):
         h = None
         kw = {}
         if read is not None:
             h = self.rt.empty(*x.shape)
             kw = dict(next_w=read[0], next_eps=read[1], h_out=h)
-        ops.post_norm_add(x, y=y, w=after.weight_f32, eps=after.eps, mult=self.mult, extra=extra, clear_y=True, y_next=y_next, **kw)
+        ops.post_norm_add(x, y=y, w=after.weight_f32, eps=after.eps, mult=self.mult if mult is None else mult, extra=extra, clear_y=True,
+                          y_next=y_next, y_bias=y_bias, **kw)
         return h
 
 

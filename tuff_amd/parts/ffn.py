@@ -231,21 +231,32 @@ class MoE(FeedForward):
     choice runs on sigmoid(z) + correction ('correction' [E], which the weights do not see) and only inside the
     route_keep groups, of route_groups equal groups of neighbouring experts, whose two largest such scores have the
     largest sum (an expert outside them cannot be chosen, whatever its score); the weights are the chosen experts'
-    sigmoid(z) times route_scale, not renormalised."""
+    sigmoid(z) times route_scale, not renormalised.
+    router_weights "softmax_share": the choice runs on s + correction with s the softmax over all outputs of the router, the
+    weights are the chosen ones' s without the correction, divided by their sum.
+    identity: the router's last `identity` outputs are identity experts, whose output is their input and which have no
+    tensors ('router' and 'correction' then have num_experts + identity rows)."""
     graph_safe = True
     records_portions = True
 
     def __init__(self, hidden_size: int, num_experts: int, top: int, expert_dim: int, *, names: dict,
                  activation: str = "relu2", router_weights: str = "sigmoid", scale_input: bool = True,
                  shared_dim: int = 0, gated: bool = False, limit: float = 0.0, alpha: float = 1.0,
-                 shared: FeedForward | None = None, route_groups: int = 0, route_keep: int = 0, route_scale: float = 1.0):
+                 shared: FeedForward | None = None, route_groups: int = 0, route_keep: int = 0, route_scale: float = 1.0,
+                 identity: int = 0):
         self.d, self.E, self.top, self.F = int(hidden_size), int(num_experts), int(top), int(expert_dim)
-        if not 1 <= self.top <= self.E:
-            raise ValueError(f"top {self.top} of {self.E} experts")
+        self.N = self.E + int(identity)                          # the router's outputs that a choice may fall on
+        if not 1 <= self.top <= self.N:
+            raise ValueError(f"top {self.top} of {self.N} experts")
+        if self.N != self.E and router_weights == "sigmoid":
+            raise ValueError("identity experts go with weights from a softmax")
         self.has_correction = "correction" in names
         self.route_scale = float(route_scale)
         self.route_groups, self.route_keep = int(route_groups), int(route_keep)
-        if not self.route_groups and (self.has_correction or self.route_scale != 1.0):
+        share = router_weights == "softmax_share"
+        if share and (self.route_groups or self.route_scale != 1.0):
+            raise ValueError("shares of the softmax go with no groups and no factor")
+        if not self.route_groups and not share and (self.has_correction or self.route_scale != 1.0):
             self.route_groups = self.route_keep = 1              # one group of all experts, kept: the choice is not limited
         if self.route_groups:
             G, keep = self.route_groups, self.route_keep
@@ -279,13 +290,13 @@ class MoE(FeedForward):
         self.shared_down = Linear(self.names["shared.down"], width, self.d)
 
     def weight_decls(self):
-        decls = [WeightDecl(self.names["router"], (self.E, self.d), "normal", role="projection")]
+        decls = [WeightDecl(self.names["router"], (self.N, self.d), "normal", role="projection")]
         if self.shared_gate:
             decls.append(WeightDecl(self.names["shared.sg"], (1, self.d), "normal", role="projection"))
         if self.has_router_bias:
-            decls.append(WeightDecl(self.names["router.b"], (self.E,), "normal"))
+            decls.append(WeightDecl(self.names["router.b"], (self.N,), "normal"))
         if self.has_correction:
-            decls.append(WeightDecl(self.names["correction"], (self.E,), "normal"))
+            decls.append(WeightDecl(self.names["correction"], (self.N,), "normal"))
         for e in self.names["experts"]:
             decls += [WeightDecl(n, (self.F, self.d), "normal", role="projection") for n in e[:-1]]
             decls.append(WeightDecl(e[-1], (self.d, self.F), "normal", role="projection"))
@@ -338,7 +349,7 @@ class MoE(FeedForward):
         z = torch.empty(T, self.router_w.shape[0], dtype=torch.float32, device=h.device)        # [T, E (+ 1)]
         ids = torch.empty(T, self.top, dtype=torch.int32, device=h.device)
         wts = torch.empty(T, self.top, dtype=torch.float32, device=h.device)
-        ops.moe_router(h, self.router_w, z, ids, wts, E=self.E, top=self.top, weights=self.router_weights, bias=self.router_b,
+        ops.moe_router(h, self.router_w, z, ids, wts, E=self.N, top=self.top, weights=self.router_weights, bias=self.router_b,
                        correction=self.correction, groups=self.route_groups, keep=self.route_keep, scale=self.route_scale)
         form = dict(activation=self.activation, scale_input=self.scale_input, gated=self.gated, limit=self.limit, alpha=self.alpha)
         if self.grouped:
@@ -352,7 +363,7 @@ class MoE(FeedForward):
             a = self.shared_up.forward(h)
             # the gate is one number a token and the second product is linear: it goes onto the activations
             if self.shared_gate:
-                ops.act_rows(a, a, self.activation, row_gate=z, gate_col=self.E, gate_activation="sigmoid")
+                ops.act_rows(a, a, self.activation, row_gate=z, gate_col=self.N, gate_activation="sigmoid")
             else:
                 ops.act_rows(a, a, self.activation)
             self.shared_down.forward(a, accumulate_into=residual)
