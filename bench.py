@@ -448,6 +448,32 @@ def kinelix_config_like(size: str):
                              "norm": {"eps": 1e-5}, "layers": layers})
 
 
+def tobilorn_config(size: str):
+    """`--design tobilorn`: half as many layers as the size has, run twice in a row, each with differential attention (half the
+    heads, each of two maps of 64 over values of 128, a window of 1,024 that keeps 4 first tokens), gated experts with two
+    identity experts beside and a shared one, and a token's own vector of an eighth of the width."""
+    from tuff_amd.models.registry import config_from_dict
+    d, L, H, G, _, E, top, eff = DESIGN_SIZES[size]
+    m = {"heads": H // 2, "kv_heads": G // 2, "dim": 64, "vdim": 128, "scale": 0.125, "diff": 0.3, "mask": {"size": 1024, "keep_first": 4},
+         "rot": {"base": 10000.0, "dims": 64}}
+    moe = {"kind": "moe", "router": {"experts": E, "top": top, "identity": 2}, "expert": {"ff": eff}, "shared": {"ff": eff}}
+    return config_from_dict({"architecture": "Tobilorn", "vocab": DESIGN_VOCAB, "width": d, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0},
+                             "token_side": {"dim": d // 8}, "loop": {"start": 0, "stop": L // 2, "times": 2},
+                             "layers": [{"type": "attention", "mixer": m, "mlp": moe}] * (L // 2)})
+
+
+def kugalorn_config_like(size: str):
+    """The Kugalorn model of the same width that tobilorn_config stands beside: one residual stream, as many layers run twice in
+    a row, window attention in every one with as many softmax maps (heads of 64, a window of 1,024, the same q, k and v
+    widths), the same experts and shared expert."""
+    from tuff_amd.models.registry import config_from_dict
+    d, L, H, G, _, E, top, eff = DESIGN_SIZES[size]
+    moe = {"kind": "moe", "router": {"experts": E, "top": top}, "expert": {"ff": eff, "limit": 7.0}, "shared": {"ff": eff, "limit": 7.0}}
+    m = {"heads": H, "kv_heads": G, "dim": 64, "vdim": 64, "scale": 0.125, "mask": {"size": 1024}}
+    return config_from_dict({"architecture": "Kugalorn", "vocab": DESIGN_VOCAB, "width": d, "norm": {"eps": 1e-6},
+                             "loop": {"start": 0, "stop": L // 2, "times": 2}, "layers": [{"type": "attention", "mixer": m, "mlp": moe}] * (L // 2)})
+
+
 def lfm2_config_like(size: str, attention_every: int = 4):
     """The LFM2 model of the same width, depth, heads, vocabulary and dense feed-forward: its short-conv
     layers stand where the other design has its recurrences (attention_every 1: attention in every layer, beside a
@@ -528,15 +554,16 @@ def time_design(cfg, dtype: str, prefill_tokens: int, batch: int, context: int, 
 
 
 def run_design(args) -> dict:
-    """`--design pafodra|kugalorn|loluzen|kinelix|kisutar`: that decoder at sizes that resemble a real model's layers (random
-    weights) beside the LFM2 decoder of equal width, depth and feed-forward (kisutar: beside the Kinelix decoder with latent
-    attention in every layer)."""
+    """`--design pafodra|kugalorn|loluzen|kinelix|kisutar|tobilorn`: that decoder at sizes that resemble a real model's layers
+    (random weights) beside the LFM2 decoder of equal width, depth and feed-forward (kisutar: beside the Kinelix decoder with
+    latent attention in every layer; tobilorn: beside the Kugalorn decoder with window attention in every layer)."""
     dtype = "bfloat16" if args.dtype == "bf16" else "float32"
     classes = os.environ.get("TUFF_TRACE", "")[:1] == "1"
     design, make = args.design, {"pafodra": pafodra_config, "kugalorn": kugalorn_config, "loluzen": loluzen_config,
-                                 "kinelix": kinelix_config, "kisutar": kisutar_config}[args.design]
+                                 "kinelix": kinelix_config, "kisutar": kisutar_config, "tobilorn": tobilorn_config}[args.design]
     every = 1 if design == "loluzen" else 4
-    other, make_other = ("kinelix", kinelix_config_like) if design == "kisutar" else ("lfm2", lambda size: lfm2_config_like(size, every))
+    beside = {"kisutar": ("kinelix", kinelix_config_like), "tobilorn": ("kugalorn", kugalorn_config_like)}
+    other, make_other = beside.get(design, ("lfm2", lambda size: lfm2_config_like(size, every)))
     out = {"design": design, "dtype": args.dtype, "prefill_tokens": PREFILL_TOKENS, "decode_batch": args.batch,
            "decode_context": args.design_context, "data": f"synthetic: seeded random weights (seed {SEED}), uniform random token ids",
            "sizes": {}}
@@ -628,9 +655,9 @@ def main() -> int:
     ap.add_argument("--shape", default="1.2b", choices=["1.2b"] + sorted(OTHER_SHAPES),
                     help="measure another shape of the architecture in the benchmark's place (for profiling; "
                          "its points only, no other shapes after it)")
-    ap.add_argument("--design", choices=["pafodra", "kugalorn", "loluzen", "kinelix", "kisutar"],
+    ap.add_argument("--design", choices=["pafodra", "kugalorn", "loluzen", "kinelix", "kisutar", "tobilorn"],
                     help="instead of the benchmark: prefill and decode of another design at sizes that resemble a real "
-                         "model's layers, beside the LFM2 model of equal size, kisutar beside Kinelix (TUFF_TRACE=1 adds GPU time by kernel class)")
+                         "model's layers, beside the LFM2 model of equal size, kisutar beside Kinelix, tobilorn beside Kugalorn (TUFF_TRACE=1 adds GPU time by kernel class)")
     ap.add_argument("--design-sizes", default="1k,2k", help="with --design: which of " + ",".join(sorted(DESIGN_SIZES)))
     ap.add_argument("--design-context", type=int, default=2048, help="with --design: tokens every decoding request holds")
     ap.add_argument("--scenario", choices=sorted(SCENARIOS),

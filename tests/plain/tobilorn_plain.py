@@ -110,7 +110,8 @@ def attention(n, W, m, eps, rnd=_same):
 def route(n, W, router, margins_out=None):
     """ids [T, top] and weights [T, top]: the largest of the softmax over all outputs plus the correction (the lower
     index wins a tie), and the chosen ones' softmax without it, divided by their sum.  margins_out: a list that
-    receives, per token, the gap between the last chosen score and the first left out (infinite where all are)."""
+    receives, per token, the gap between the last chosen score and the first left out as a share of their softmax scores
+    (infinite where all are chosen)."""
     N, top = router["experts"] + router.get("identity", 0), router["top"]
     z = n @ W["router"].T
     s = torch.exp(z - z.max(-1, keepdim=True).values)
@@ -123,7 +124,8 @@ def route(n, W, router, margins_out=None):
         order = sorted(range(N), key=lambda e: (-c[t, e].item(), e))
         ids[t] = torch.tensor(order[:top])
         if top < N:
-            margins[t] = c[t, order[top - 1]] - c[t, order[top]]
+            a, b = order[top - 1], order[top]
+            margins[t] = (c[t, a] - c[t, b]) / (s[t, a] + s[t, b])
     if margins_out is not None:
         margins_out.append(margins)
     w = torch.gather(s, 1, ids)

@@ -49,6 +49,49 @@ def test_groups_by_window_and_shared_page_numbering():
         CacheLayout.from_specs({0: "ring buffer"})
 
 
+def test_groups_by_window_and_first_tokens_that_stay():
+    lay = CacheLayout.from_specs({0: PagedKV(2, 16, 32, keep_first=4), 1: PagedKV(2, 16, 32), 2: PagedKV(1, 8, 32, keep_first=4),
+                                  3: PagedKV(1, 8, keep_first=9), 4: PagedKV(1, 8)})
+    assert list(zip(lay.group_windows, lay.group_keeps)) == [(32, 4), (32, 0), (None, 0)]     # without a window everything stays anyway
+    assert lay.group_of_entry == {0: 0, 1: 1, 2: 0, 3: 2, 4: 2}
+
+
+@pytest.mark.parametrize("keep", [0, 1, 4, 5, 8, 13, 40])
+@pytest.mark.parametrize("window", [1, 4, 6, 17])
+def test_a_window_gives_back_what_it_has_passed_but_not_the_first_tokens_that_stay(window, keep):
+    """After every step exactly the pages are held that a later token still reads: every position that the next token (or
+    any after it) sees lies in a held page, and no page is held all of whose positions none of them sees."""
+    ps = 4
+    lay = CacheLayout.from_specs({0: PagedKV(1, 8, window, keep_first=keep)})
+    m = CacheManager(lay, ps, 64, 2)
+    m.admit("other")
+    m.extend("other", 3)
+    rng = random.Random(window * 100 + keep)
+    m.admit("a")
+    while m.length("a") < 90:
+        back = m.reclaimable("a")[0]
+        free = m.groups[0].pool.num_free
+        n = rng.choice([1, 1, 2, 3, 7])
+        need = m.pages_needed("a", n)[0]
+        before = m.length("a")
+        m.extend("a", n)
+        assert m.groups[0].pool.num_free == free + back - need
+        m.check()
+        table = m.block_table("a", 0)
+        # what extend() keeps: positions its own tokens read, the earliest of which is the first new token's
+        read = {j for i in range(before, m.length("a")) for j in range(i + 1) if i - j < window or j < keep}
+        for b, page in enumerate(table):
+            here = set(range(b * ps, (b + 1) * ps))
+            later = any(i - j < window or j < keep for j in here for i in range(before, before + 1 + window) if j <= i)
+            assert (page != FREED) == (later or b * ps >= before - before % ps), (before, b)
+            if here & read:
+                assert page != FREED
+    m.release("a")
+    m.release("other")
+    m.check()
+    assert m.groups[0].pool.num_free == 64
+
+
 def test_extend_release_and_lookup():
     m = CacheManager(layout(), page_size=4, num_pages=6, num_slots=2)
     s = m.admit("a")

@@ -112,6 +112,8 @@ def make_weights(raw: dict, seed: int) -> dict:
             t = n(0.6 / math.sqrt(math.sqrt(shape[0])))
         elif last == "correction":
             t = n(0.1)
+        elif name.endswith("side.gate"):                  # it reads the stream as it is: an activation in its curved part
+            t = n(1.3 / math.sqrt(shape[1]) / max(1.0, raw["embedding"]["scale"]))
         elif last == "router":
             t = n(1.5 / math.sqrt(shape[1]))
         elif len(shape) == 2:

@@ -90,11 +90,14 @@ def _inspect(cfg, model, out=sys.stdout) -> None:
     for i, b in enumerate(model.blocks):
         # a block of another arrangement may have neither a mixer nor a feed-forward of these names
         mixer, ffn = getattr(b, "mixer", None), getattr(b, "ffn", None)
-        inside = " + ".join(_part_name(p) for p in (mixer, ffn) if p is not None) or type(b).__name__
+        inside = " + ".join(_part_name(p) for p in (mixer, ffn, getattr(b, "side", None)) if p is not None) or type(b).__name__
         spec = mixer.cache_spec() if hasattr(mixer, "cache_spec") else None
         own = b.block_state() if hasattr(b, "block_state") else None
         print(f"  layer {i}: {type(b).__name__}: {inside}  cache: {spec}" + (f"  own state: {own}" if own is not None else ""), file=out)
     print(f"run order: {[r.block for r in model.schedule]}", file=out)
+    begins = [i for i, r in enumerate(model.schedule) if getattr(r, "enter", None) is not None]
+    if begins:
+        print(f"  passes begin with {type(model.entry).__name__} before runs {begins}", file=out)
 
 
 def main(argv=None) -> int:
