@@ -136,6 +136,85 @@ __global__ __launch_bounds__(PN_THREADS) void post_norm_add_regs_kernel(
     }
 }
 
+// The same for rows of a multiple of four elements, up to 4,096: a thread holds VPT times four neighbouring ones, a workgroup
+// has as many waves as the row needs, so a row's few loads are 16 bytes wide and all under way at once, which is what a step
+// of few tokens waits for.  Sums: a thread's elements in ascending order, the butterfly of a wave, the waves in order.
+constexpr int PN_VEC_MAX = 4096;
+
+__device__ __forceinline__ float waves_sum(float v, float* scratch, int waves) {
+    v = wave_sum(v);
+    if (threadIdx.x % WAVE == 0) scratch[threadIdx.x / WAVE] = v;
+    __syncthreads();
+    float t = 0.f;
+    for (int i = 0; i < waves; ++i) t += scratch[i];
+    return t;
+}
+
+template <typename T, int VPT>
+__global__ __launch_bounds__(PN_VEC_MAX / 4 / VPT) void post_norm_add_vec_kernel(
+    float* __restrict__ x, float* __restrict__ y, const float* __restrict__ w, float eps, float mult,
+    const float* __restrict__ extra, const float* __restrict__ w_next, float eps_next, T* __restrict__ h_out,
+    int d, int clear_y, const float* __restrict__ y_next, const float* __restrict__ y_bias, const float* __restrict__ row_add) {
+    typedef T out4 __attribute__((ext_vector_type(4)));
+    __shared__ float scratch[2][PN_VEC_MAX / 4 / WAVE];
+    const int waves = blockDim.x / WAVE;
+    const long long row = (long long)blockIdx.x * d;
+    const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+    f32x4 xv[VPT], yv[VPT], wv[VPT], ev[VPT], rv[VPT], nv[VPT];
+    auto place = [&](int k) { return (int)(threadIdx.x + k * blockDim.x) * 4; };
+#pragma unroll
+    for (int k = 0; k < VPT; ++k) {
+        const int c = place(k);
+        const bool in = c < d;
+        xv[k] = in ? *(const f32x4*)(x + row + c) : zero;
+        yv[k] = (in && y) ? *(const f32x4*)(y + row + c) : zero;
+        wv[k] = (in && y) ? *(const f32x4*)(w + c) : zero;
+        if (in && y_bias) yv[k] += *(const f32x4*)(y_bias + c);
+        ev[k] = (in && extra) ? *(const f32x4*)(extra + row + c) : zero;
+        rv[k] = (in && row_add) ? *(const f32x4*)(row_add + c) : zero;
+        nv[k] = (in && w_next) ? *(const f32x4*)(w_next + c) : zero;
+    }
+    if (y) {
+        float ss = 0.f;
+#pragma unroll
+        for (int k = 0; k < VPT; ++k)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) ss = fmaf(yv[k][e], yv[k][e], ss);
+        ss = waves_sum(ss, scratch[0], waves);
+        const float inv = mult / sqrtf(ss / (float)d + eps);
+#pragma unroll
+        for (int k = 0; k < VPT; ++k) {
+            const int c = place(k);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) xv[k][e] = fmaf(yv[k][e] * inv, wv[k][e], xv[k][e]);
+            if (c < d && clear_y) *(f32x4*)(y + row + c) = y_next ? *(const f32x4*)(y_next + c) : zero;
+        }
+    }
+    float ss2 = 0.f;
+#pragma unroll
+    for (int k = 0; k < VPT; ++k) {
+        const int c = place(k);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            if (extra) xv[k][e] += ev[k][e];
+            if (row_add) xv[k][e] += rv[k][e];
+            ss2 = fmaf(xv[k][e], xv[k][e], ss2);
+        }
+        if (c < d && (y || extra || row_add)) *(f32x4*)(x + row + c) = xv[k];
+    }
+    if (!h_out) return;
+    float inv2 = 1.0f;
+    if (w_next) inv2 = 1.0f / sqrtf(waves_sum(ss2, scratch[1], waves) / (float)d + eps_next);
+#pragma unroll
+    for (int k = 0; k < VPT; ++k) {
+        const int c = place(k);
+        out4 o;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] = from_f32<T>(w_next ? xv[k][e] * inv2 * nv[k][e] : xv[k][e]);
+        if (c < d) *(out4*)(h_out + row + c) = o;
+    }
+}
+
 __global__ __launch_bounds__(PN_THREADS) void normed_mean2_kernel(
     const float* __restrict__ a, const float* __restrict__ wa, const float* __restrict__ b, const float* __restrict__ wb,
     float eps, float coef, float* __restrict__ out, int d) {
@@ -249,7 +328,21 @@ TUFF_EXPORT int tuff_post_norm_add(float* x, float* y, const float* w, float eps
     if (n_tokens <= 0) return 0;
     if (d <= 0 || (y && !w) || (w_next && !h_out) || (y_bias && !y)) return -2;
     dim3 grid(n_tokens), block(PN_THREADS);
+    // (rows and weights lie on 16-byte borders where the row's width is a multiple of four: the caller's tensors start on them)
+    const uintptr_t ends = (uintptr_t)x | (uintptr_t)y | (uintptr_t)w | (uintptr_t)extra | (uintptr_t)w_next | (uintptr_t)h_out |
+                           (uintptr_t)y_next | (uintptr_t)y_bias | (uintptr_t)row_add;
+    const bool vec = d % 4 == 0 && d <= PN_VEC_MAX && ends % 16 == 0;
+    const int vpt = d > 1024 ? 2 : 1;
+    if (vec) block = dim3(ceil_div(ceil_div(d / 4, vpt), WAVE) * WAVE);
 #define LAUNCH(KERN, T) hipLaunchKernelGGL(KERN, grid, block, 0, stream, x, y, w, eps, mult, extra, w_next, eps_next, (T*)h_out, d, clear_y, y_next, y_bias, row_add)
+    if (vec) {
+        if (vpt == 1) {
+            if (out_dt == DT_F32) LAUNCH((post_norm_add_vec_kernel<float, 1>), float); else LAUNCH((post_norm_add_vec_kernel<bf16_t, 1>), bf16_t);
+        } else {
+            if (out_dt == DT_F32) LAUNCH((post_norm_add_vec_kernel<float, 2>), float); else LAUNCH((post_norm_add_vec_kernel<bf16_t, 2>), bf16_t);
+        }
+        return launch_status();
+    }
     if (d <= PN_THREADS * 8) {
         if (out_dt == DT_F32) LAUNCH((post_norm_add_regs_kernel<float, 8>), float); else LAUNCH((post_norm_add_regs_kernel<bf16_t, 8>), bf16_t);
     } else if (d <= PN_THREADS * 32) {
